@@ -306,6 +306,7 @@ class LatentAttentionConfig:
     rot_base: float
     scale: float
     kv_from: int = -1
+    window: int = 0   # sliding window (Kolotar); 0: every earlier key
 
 
 @dataclass(frozen=True)
@@ -768,6 +769,199 @@ HYBRID_PRESETS.update({
                                        1024, 8, 2, 7168, 0, 2, 1, 3584),
 })
 ARCHITECTURES["Lovapel"] = LovapelConfig.from_dict
+
+
+# ---------------------------------------------------------------------------------------
+# Kolotar: post-norm decoder (the residual itself is normed after every sum) whose layers pick
+# one of three mixers - gated window attention with a sink and mixed values, window latent
+# attention, or sigmoid attention with talking heads next to a gated delta rule - followed by
+# routed experts.
+
+@dataclass(frozen=True)
+class GatedWindowAttentionConfig:
+    """Grouped-query softmax attention with biased projections, per-head q / k RMS norm before
+    rotate-half positions on the first ``rot_dims`` channels (YaRN ``rot_scaling`` = (factor,
+    original, fast, slow)), values divided by their root mean square per head, a sliding window
+    of ``window`` keys (0: all earlier keys), one learned sink score per query head and a
+    sigmoid output gate per head.  ``v_mix``: the values of every such layer but the first are
+    mixed with the first one's values of the same token."""
+    heads: int
+    kv_heads: int
+    dim: int
+    vdim: int
+    scale: float
+    window: int = 0
+    rot_dims: int = 0
+    rot_base: float = 10000.0
+    rot_scaling: tuple | None = None
+    v_mix: bool = False
+
+
+@dataclass(frozen=True)
+class SigmoidMixerConfig:
+    """Grouped-query attention whose weights are sigmoids (soft-capped score plus a number per
+    head), not normalised over the keys and mixed across the heads by a [heads, heads] matrix; q
+    and k normed over their whole projection, no rotation, q scaled by
+    1 + temp_coef ln(floor((position + 1) / temp_every) + 1)."""
+    heads: int
+    kv_heads: int
+    dim: int
+    vdim: int
+    scale: float
+    softcap: float = 0.0
+    temp_coef: float = 0.0
+    temp_every: float = 1.0
+
+
+@dataclass(frozen=True)
+class TopMoeConfig:
+    """``experts`` SiLU-GLU feed-forward layers of width ``ff``; a token runs the ``top`` with the
+    largest router logits, weighted by the softmax over those."""
+    experts: int
+    top: int
+    ff: int
+
+
+@dataclass(frozen=True)
+class KolotarLayerConfig:
+    kind: str                 # "attention" | "latent_attention" | "parallel"
+    mixer: object = None      # parallel: the left branch (SigmoidMixerConfig)
+    delta: DeltaMixerConfig | None = None     # parallel: the right branch
+    left_scale: float = 1.0
+    right_scale: float = 1.0
+    moe: TopMoeConfig | None = None           # None: no feed-forward
+
+
+@dataclass(frozen=True)
+class KolotarConfig:
+    name: str = "kolotar"
+    vocab_size: int = 1024
+    hidden_size: int = 256
+    layers: tuple = ()
+    rms_norm_eps: float = 1e-5
+    alpha: float = 1.0        # weight of the residual inside every post-norm
+    bos_token_id: int = 0
+    eos_token_ids: tuple = ()
+    max_position_embeddings: int = 1 << 20
+    family: str = "kolotar"
+
+    @property
+    def num_layers(self) -> int:
+        return len(self.layers)
+
+    @property
+    def first_v_mix(self) -> int:
+        """Index of the layer whose values the later ``v_mix`` layers mix in (-1: none)."""
+        for i, L in enumerate(self.layers):
+            if L.kind == "attention" and L.mixer.v_mix:
+                return i
+        return -1
+
+    def __post_init__(self):
+        shapes = {(L.mixer.kv_heads, L.mixer.vdim) for L in self.layers
+                  if L.kind == "attention" and L.mixer.v_mix}
+        if len(shapes) > 1:
+            raise ValueError("layers that mix values need the same kv_heads and vdim")
+
+    @staticmethod
+    def from_dict(c: dict, name: str = "kolotar") -> "KolotarConfig":
+        """Parse the checkpoint's config.json (keys: vocab, width, norm.eps, postln_alpha,
+        layers[].{type, mixer, mlp}; attention: heads, kv_heads, dim, vdim, scale, mask.size,
+        rot.{dims, base, scaling.{factor, original, fast, slow}}, v_mix; latent_attention: heads,
+        dim, rot_dim, vdim, kv_rank, scale, mask.size, rot.{dims, base}; parallel: left.{heads,
+        kv_heads, dim, vdim, scale, softcap, q_temp.{coef, every}}, right.{heads, kv_heads, dim,
+        vdim, conv}, left_scale, right_scale; mlp: kind moe {expert.ff, router.{experts, top}} or
+        null).  An absent mask, rot, scaling, softcap, q_temp or v_mix means none."""
+
+        def heads(m, i):
+            h, g = int(m["heads"]), int(m.get("kv_heads", m["heads"]))
+            if g < 1 or h % g:
+                raise ValueError(f"layer {i}: heads must be a multiple of kv_heads")
+            return {"heads": h, "kv_heads": g, "dim": int(m["dim"]),
+                    "vdim": int(m.get("vdim", m["dim"]))}
+
+        layers = []
+        for i, L in enumerate(c["layers"]):
+            m, t = L["mixer"], L["type"]
+            kw = {}
+            if t in ("attention", "latent_attention"):
+                rot = m.get("rot") or {}
+                sc = rot.get("scaling")
+                window = int((m.get("mask") or {}).get("size") or 0)
+                rot_dims, base = int(rot.get("dims", 0)), float(rot.get("base", 10000.0))
+                width = int(m["dim"] if t == "attention" else m["rot_dim"])
+                if rot_dims % 2 or rot_dims > width:
+                    raise ValueError(f"layer {i}: rot.dims must be even and <= {width}")
+            if t == "attention":
+                mc = GatedWindowAttentionConfig(
+                    **heads(m, i), scale=float(m["scale"]), window=window, rot_dims=rot_dims,
+                    rot_base=base,
+                    rot_scaling=(float(sc["factor"]), float(sc["original"]), float(sc["fast"]),
+                                 float(sc["slow"])) if sc else None,
+                    v_mix=bool(m.get("v_mix", False)))
+            elif t == "latent_attention":
+                mc = LatentAttentionConfig(
+                    heads=int(m["heads"]), dim=int(m["dim"]), rot_dim=int(m["rot_dim"]),
+                    vdim=int(m["vdim"]), kv_rank=int(m["kv_rank"]), q_rank=0, rot_dims=rot_dims,
+                    rot_base=base, scale=float(m["scale"]), window=window)
+            elif t == "parallel":
+                a, d = m["left"], m["right"]
+                qt = a.get("q_temp") or {}
+                mc = SigmoidMixerConfig(
+                    **heads(a, i), scale=float(a["scale"]), softcap=float(a.get("softcap") or 0.0),
+                    temp_coef=float(qt.get("coef", 0.0)), temp_every=float(qt.get("every", 1.0)))
+                kw = {"delta": DeltaMixerConfig(**heads(d, i), conv=int(d["conv"])),
+                      "left_scale": float(m["left_scale"]), "right_scale": float(m["right_scale"])}
+            else:
+                raise ValueError(f"unknown layer type {t!r}")
+            mlp = L.get("mlp")
+            if mlp:
+                kind = str(mlp.get("kind", "moe"))
+                if kind != "moe":
+                    raise ValueError(f"unsupported feed-forward kind {kind!r}")
+                kw["moe"] = TopMoeConfig(experts=int(mlp["router"]["experts"]),
+                                         top=int(mlp["router"]["top"]), ff=int(mlp["expert"]["ff"]))
+                if not 1 <= kw["moe"].top <= kw["moe"].experts:
+                    raise ValueError(f"layer {i}: router.top must be in [1, experts]")
+            layers.append(KolotarLayerConfig(t, mc, **kw))
+        return KolotarConfig(name=name, vocab_size=int(c["vocab"]), hidden_size=int(c["width"]),
+                             layers=tuple(layers), rms_norm_eps=float(c["norm"]["eps"]),
+                             alpha=float(c["postln_alpha"]))
+
+
+def kolotar_preset(name: str, vocab: int, width: int, ff: int, pattern: str, heads: int,
+                   kv_heads: int, dim: int, kv_rank: int, window: int, experts: int = 8,
+                   top: int = 2, rot_dim: int = 64) -> KolotarConfig:
+    """A Kolotar shape for benchmarks and tests: one letter per layer, ``a`` gated window
+    attention, ``l`` latent attention, ``p`` sigmoid attention next to a delta rule; every layer
+    has ``experts`` experts of width ``ff``."""
+    moe = TopMoeConfig(experts, top, ff)
+    att = GatedWindowAttentionConfig(heads, kv_heads, dim, dim, dim ** -0.5, window, dim, 500000.0,
+                                     (4.0, 4096.0, 32.0, 1.0), True)
+    lat = LatentAttentionConfig(heads, dim, rot_dim, dim, kv_rank, 0, rot_dim, 10000.0,
+                                (dim + rot_dim) ** -0.5, window=window)
+    sig = SigmoidMixerConfig(heads, kv_heads, dim, dim, dim ** -0.5, 15.0, 0.1, 1024.0)
+    dlt = DeltaMixerConfig(heads, kv_heads, dim, dim, 4)
+    made = {"a": KolotarLayerConfig("attention", att, moe=moe),
+            "l": KolotarLayerConfig("latent_attention", lat, moe=moe),
+            "p": KolotarLayerConfig("parallel", sig, dlt, 0.7, 0.8, moe)}
+    return KolotarConfig(name=name, vocab_size=vocab, hidden_size=width,
+                         layers=tuple(made[ch] for ch in pattern), alpha=1.5)
+
+
+HYBRID_PRESETS.update({
+    "kolotar-tiny": kolotar_preset("kolotar-tiny", 512, 128, 48, "palpa", 4, 2, 32, 48, 24, 6, 2,
+                                   16),
+    # the "small" Llama preset's geometry (width 1024, 8 q / 2 kv heads of 128, FFN 2816, 4 layers)
+    "kolotar-small": kolotar_preset("kolotar-small", 32768, 1024, 1408, "alpa", 8, 2, 128, 192,
+                                    1024),
+    # Llama-3.2-3B / Llama-3.1-8B layer geometry, one layer per mixer
+    "kolotar-3b-slice": kolotar_preset("kolotar-3b-slice", 16384, 3072, 4096, "alp", 24, 8, 128,
+                                       192, 1024),
+    "kolotar-8b-slice": kolotar_preset("kolotar-8b-slice", 16384, 4096, 7168, "alp", 32, 8, 128,
+                                       192, 1024),
+})
+ARCHITECTURES["Kolotar"] = KolotarConfig.from_dict
 
 
 def resolve_model(model: str) -> tuple[ModelConfig, str | None]:

@@ -23,7 +23,11 @@ def model_class(family: str):
         from .lovapel import LovapelModel
 
         return LovapelModel
+    if family == "kolotar":
+        from .kolotar import KolotarModel
+
+        return KolotarModel
     raise ValueError(f"no model registered for family {family!r}")
 
 
-FAMILIES = ("llama", "ledazen", "soselix", "semezen", "lovapel")
+FAMILIES = ("llama", "ledazen", "soselix", "semezen", "lovapel", "kolotar")

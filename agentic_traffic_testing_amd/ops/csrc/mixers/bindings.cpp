@@ -156,7 +156,9 @@ void qk_norm_rope_cache(at::Tensor q_out, const at::Tensor& qx, const at::Tensor
                         const at::Tensor& positions, const at::Tensor& slot_mapping,
                         const at::Tensor& cos_sin, at::Tensor k_cache, at::Tensor v_cache,
                         bool rotate_half, bool norm_last,
-                        const c10::optional<at::Tensor>& row_inv) {
+                        const c10::optional<at::Tensor>& row_inv, double temp_coef,
+                        double temp_every, bool v_norm, const c10::optional<at::Tensor>& v_first,
+                        double v_lambda, const c10::optional<at::Tensor>& v_out) {
   TORCH_CHECK(q_out.dim() == 3 && q_out.is_contiguous() && k_cache.dim() == 4 &&
                   v_cache.dim() == 4 && k_cache.is_contiguous() && v_cache.is_contiguous(),
               "qk_norm_rope_cache: q_out [T, H, d], caches [nb, G, BS, d]");
@@ -185,6 +187,13 @@ void qk_norm_rope_cache(at::Tensor q_out, const at::Tensor& qx, const at::Tensor
     f32c(*row_inv, "row_inv");
     TORCH_CHECK(row_inv->numel() == 2 * T && !norm_last, "qk_norm_rope_cache: row_inv [T, 2]");
   }
+  TORCH_CHECK(temp_coef == 0.0 || (temp_every > 0.0 && !norm_last),
+              "qk_norm_rope_cache: a query temperature needs every > 0 and the norm first");
+  for (const auto* v : {&v_first, &v_out})
+    if (v->has_value())
+      TORCH_CHECK((*v)->is_cuda() && (*v)->is_contiguous() && (*v)->numel() == T * G * vdim &&
+                      (*v)->scalar_type() == q_out.scalar_type(),
+                  "qk_norm_rope_cache: v_first / v_out [T, G * vdim]");
   int64_t heads_of = H;
   for (const auto* w : {&q_norm, &k_norm}) {
     if (w->has_value())
@@ -201,12 +210,16 @@ void qk_norm_rope_cache(at::Tensor q_out, const at::Tensor& qx, const at::Tensor
                                 positions.data_ptr<int>(), slot_mapping.data_ptr<int>(),
                                 cos_sin.data_ptr<float>(), n_freq, k_cache.data_ptr(),
                                 v_cache.data_ptr(), T, H, G, dim, vdim, BS, rotate_half, norm_last,
-                                row_inv ? row_inv->data_ptr<float>() : nullptr, code(q_out),
-                                cur_stream()),
+                                row_inv ? row_inv->data_ptr<float>() : nullptr,
+                                static_cast<float>(temp_coef), static_cast<float>(temp_every),
+                                v_norm, v_first ? v_first->data_ptr() : nullptr,
+                                static_cast<float>(v_lambda), v_out ? v_out->data_ptr() : nullptr,
+                                code(q_out), cur_stream()),
         "qk_norm_rope_cache");
 }
 
-void rotary_table(at::Tensor out, const at::Tensor& positions, const at::Tensor& inv_freq) {
+void rotary_table(at::Tensor out, const at::Tensor& positions, const at::Tensor& inv_freq,
+                  double mult) {
   i32(positions, "positions");
   f32c(inv_freq, "inv_freq");
   f32c(out, "out");
@@ -215,7 +228,8 @@ void rotary_table(at::Tensor out, const at::Tensor& positions, const at::Tensor&
               "rotary_table: out [rows, 2 n_freq]");
   const at::DeviceGuard g(out.device());
   rc_ok(mixk_rotary_table(out.data_ptr<float>(), positions.data_ptr<int>(),
-                          inv_freq.data_ptr<float>(), out.size(0), inv_freq.numel(), cur_stream()),
+                          inv_freq.data_ptr<float>(), out.size(0), inv_freq.numel(),
+                          static_cast<float>(mult), cur_stream()),
         "rotary_table");
 }
 
@@ -225,7 +239,8 @@ void sink_attention(at::Tensor out, const at::Tensor& q, const at::Tensor& k_cac
                     const at::Tensor& tile_seq, const at::Tensor& tile_qoff, double scale,
                     bool sink, int64_t num_decode, int64_t max_decode_kv,
                     const c10::optional<at::Tensor>& part, bool use_mfma,
-                    const c10::optional<at::Tensor>& sink_val, int64_t window) {
+                    const c10::optional<at::Tensor>& sink_val, int64_t window,
+                    const c10::optional<at::Tensor>& gate) {
   TORCH_CHECK(q.is_cuda() && q.dim() == 3 && q.is_contiguous() && out.dim() == 3 &&
                   out.is_contiguous() && k_cache.dim() == 4 && v_cache.dim() == 4 &&
                   k_cache.is_contiguous() && v_cache.is_contiguous(),
@@ -270,6 +285,10 @@ void sink_attention(at::Tensor out, const at::Tensor& q, const at::Tensor& k_cac
     TORCH_CHECK(sink && sink_val->numel() == H, "sink_attention: sink_val [H] needs sink");
     sink_ptr = sink_val->data_ptr<float>();
   }
+  if (gate) {
+    rows2d(*gate, q, "gate");
+    TORCH_CHECK(gate->size(0) == q.size(0) && gate->size(1) == H, "sink_attention: gate [T, H]");
+  }
   const at::DeviceGuard g(q.device());
   rc_ok(mixk_sink_attention(out.data_ptr(), q.data_ptr(), k_cache.data_ptr(), v_cache.data_ptr(),
                             block_tables.data_ptr<int>(), block_tables.size(1),
@@ -277,8 +296,62 @@ void sink_attention(at::Tensor out, const at::Tensor& q, const at::Tensor& k_cac
                             tile_seq.data_ptr<int>(), tile_qoff.data_ptr<int>(), tile_seq.numel(),
                             num_decode, max_decode_kv, part_ptr, max_parts, H, G, dim, vdim, BS,
                             static_cast<float>(scale), sink, sink_ptr, static_cast<int>(window),
+                            gate ? gate->data_ptr() : nullptr, gate ? gate->stride(0) : 0,
                             use_mfma, code(q), cur_stream()),
         "sink_attention");
+}
+
+void sigmoid_attention(at::Tensor out, const at::Tensor& q, const at::Tensor& k_cache,
+                       const at::Tensor& v_cache, const at::Tensor& block_tables,
+                       const at::Tensor& seq_kvlen, const at::Tensor& seq_qstart,
+                       const at::Tensor& tile_seq, const at::Tensor& tile_qoff, double scale,
+                       double cap, const at::Tensor& bias, const at::Tensor& talk,
+                       int64_t num_decode, int64_t max_decode_kv,
+                       const c10::optional<at::Tensor>& part, bool use_mfma) {
+  TORCH_CHECK(q.is_cuda() && q.dim() == 3 && q.is_contiguous() && out.is_cuda() &&
+                  out.dim() == 3 && out.is_contiguous() && k_cache.dim() == 4 &&
+                  v_cache.dim() == 4 && k_cache.is_contiguous() && v_cache.is_contiguous(),
+              "sigmoid_attention: q [T, H, d], out [T, H, dv], K [nb, G, BS, d], V [nb, G, dv, BS]");
+  const int64_t H = q.size(1), dim = q.size(2), G = k_cache.size(1), BS = k_cache.size(2);
+  const int64_t vdim = v_cache.size(2), S = seq_kvlen.numel();
+  i32(block_tables, "block_tables");
+  i32(seq_kvlen, "seq_kvlen");
+  i32(seq_qstart, "seq_qstart");
+  i32(tile_seq, "tile_seq");
+  i32(tile_qoff, "tile_qoff");
+  f32c(bias, "bias");
+  f32c(talk, "talk");
+  TORCH_CHECK(block_tables.dim() == 2 && block_tables.size(0) >= S &&
+                  seq_qstart.numel() == S + 1 && tile_seq.numel() == tile_qoff.numel() &&
+                  out.size(0) == q.size(0) && out.size(1) == H && out.size(2) == vdim &&
+                  k_cache.size(3) == dim && v_cache.size(1) == G && v_cache.size(3) == BS &&
+                  v_cache.size(0) == k_cache.size(0) && G > 0 && H % G == 0 &&
+                  out.scalar_type() == q.scalar_type() &&
+                  k_cache.scalar_type() == q.scalar_type() &&
+                  v_cache.scalar_type() == q.scalar_type() && num_decode >= 0 &&
+                  num_decode <= S && bias.numel() == H && talk.numel() == H * H && cap >= 0.0,
+              "sigmoid_attention: shapes");
+  float* part_ptr = nullptr;
+  int64_t max_parts = 0;
+  if (num_decode > 0) {
+    TORCH_CHECK(part.has_value(), "sigmoid_attention: decode rows need the partials workspace");
+    f32c(*part, "part");
+    TORCH_CHECK(part->dim() == 4 && part->size(0) >= num_decode && part->size(1) == H &&
+                    part->size(3) == vdim && max_decode_kv >= 1 &&
+                    part->size(2) * 64 >= max_decode_kv,
+                "sigmoid_attention: partials [num_decode, H, parts of 64 keys, vdim]");
+    part_ptr = part->data_ptr<float>();
+    max_parts = part->size(2);
+  }
+  const at::DeviceGuard g(q.device());
+  rc_ok(mixk_sigmoid_attention(
+            out.data_ptr(), q.data_ptr(), k_cache.data_ptr(), v_cache.data_ptr(),
+            block_tables.data_ptr<int>(), block_tables.size(1), seq_kvlen.data_ptr<int>(),
+            seq_qstart.data_ptr<int>(), tile_seq.data_ptr<int>(), tile_qoff.data_ptr<int>(),
+            tile_seq.numel(), num_decode, max_decode_kv, part_ptr, max_parts, H, G, dim, vdim, BS,
+            static_cast<float>(scale), static_cast<float>(cap), bias.data_ptr<float>(),
+            talk.data_ptr<float>(), use_mfma, code(q), cur_stream()),
+        "sigmoid_attention");
 }
 
 void short_conv_silu(at::Tensor out, const at::Tensor& x, const at::Tensor& w,
@@ -412,21 +485,25 @@ void head_gate(at::Tensor out, const at::Tensor& o, const at::Tensor& gate) {
   TORCH_CHECK(o.is_cuda() && o.dim() == 3 && o.is_contiguous(), "head_gate: o [H, T, dv]");
   const int64_t H = o.size(0), T = o.size(1), dv = o.size(2);
   rows2d(gate, o, "gate");
-  TORCH_CHECK(gate.size(0) == T && gate.size(1) == H && out.is_contiguous() &&
-                  out.numel() == o.numel() && out.scalar_type() == o.scalar_type(),
+  // gate [T, H]: one number per head; [T, H * dv]: one per channel
+  TORCH_CHECK(gate.size(0) == T && (gate.size(1) == H || gate.size(1) == H * dv) &&
+                  out.is_contiguous() && out.numel() == o.numel() &&
+                  out.scalar_type() == o.scalar_type(),
               "head_gate: shapes");
   const at::DeviceGuard g(o.device());
   rc_ok(mixk_head_gate(out.data_ptr(), o.data_ptr(), gate.data_ptr(), gate.stride(0), T, H, dv,
-                       code(o), cur_stream()),
+                       gate.size(1) != H, code(o), cur_stream()),
         "head_gate");
 }
 
 void latent_rope_cache(at::Tensor q_out, const at::Tensor& q_lat, const at::Tensor& qx,
                        const c10::optional<at::Tensor>& kvx, const c10::optional<at::Tensor>& c_norm,
                        double eps, const at::Tensor& slot_mapping, const at::Tensor& cos_sin,
-                       at::Tensor k_cache, at::Tensor v_cache, at::Tensor c_out) {
+                       at::Tensor k_cache, at::Tensor v_cache, at::Tensor c_out,
+                       bool rotate_half) {
   TORCH_CHECK(q_out.is_cuda() && q_out.dim() == 3 && q_out.is_contiguous() && q_lat.dim() == 3 &&
-                  q_lat.is_contiguous() && qx.dim() == 3 && qx.is_contiguous() &&
+                  q_lat.is_contiguous() && qx.is_cuda() && qx.dim() == 3 && qx.stride(2) == 1 &&
+                  (qx.size(1) == 1 || qx.stride(1) == qx.size(2)) &&
                   k_cache.dim() == 4 && v_cache.dim() == 4 && k_cache.is_contiguous() &&
                   v_cache.is_contiguous(),
               "latent_rope_cache: q_out [T, H, rank + rot], q_lat [H, T, rank], qx [T, H, qdim + rot]");
@@ -463,11 +540,11 @@ void latent_rope_cache(at::Tensor q_out, const at::Tensor& q_lat, const at::Tens
     kv_stride = kvx->stride(0);
   }
   const at::DeviceGuard g(q_out.device());
-  rc_ok(mixk_latent_rope_cache(q_out.data_ptr(), q_lat.data_ptr(), qx.data_ptr(), kv_ptr,
-                               kv_stride, norm_ptr, static_cast<float>(eps),
+  rc_ok(mixk_latent_rope_cache(q_out.data_ptr(), q_lat.data_ptr(), qx.data_ptr(), qx.stride(0),
+                               kv_ptr, kv_stride, norm_ptr, static_cast<float>(eps),
                                slot_mapping.data_ptr<int>(), cos_sin.data_ptr<float>(), n_freq,
                                k_cache.data_ptr(), v_cache.data_ptr(), c_out.data_ptr(), T, H,
-                               qdim, rank, rot, BS, code(q_out), cur_stream()),
+                               qdim, rank, rot, BS, rotate_half, code(q_out), cur_stream()),
         "latent_rope_cache");
 }
 
@@ -622,7 +699,7 @@ void mingru_scan(at::Tensor out, at::Tensor state, const at::Tensor& z, const at
         "mingru_scan");
 }
 
-void moe_route(at::Tensor idx, at::Tensor wts, const at::Tensor& logits, bool softmax,
+void moe_route(at::Tensor idx, at::Tensor wts, const at::Tensor& logits, int64_t score,
                const c10::optional<at::Tensor>& correction, int64_t groups, int64_t keep,
                bool renorm) {
   f32c(logits, "logits");
@@ -643,7 +720,7 @@ void moe_route(at::Tensor idx, at::Tensor wts, const at::Tensor& logits, bool so
   const at::DeviceGuard g(logits.device());
   rc_ok(mixk_moe_route(idx.data_ptr<int>(), wts.data_ptr<float>(), logits.data_ptr<float>(),
                        correction ? correction->data_ptr<float>() : nullptr, logits.size(0),
-                       logits.size(1), idx.size(1), softmax, groups, keep, renorm, cur_stream()),
+                       logits.size(1), idx.size(1), static_cast<int>(score), groups, keep, renorm, cur_stream()),
         "moe_route");
 }
 
@@ -763,6 +840,30 @@ void norm_add_norm(const c10::optional<at::Tensor>& h, at::Tensor x,
         "norm_add_norm");
 }
 
+void post_norm(const c10::optional<at::Tensor>& h, at::Tensor x, double alpha, const at::Tensor& a,
+               double sa, const c10::optional<at::Tensor>& b, double sb, const at::Tensor& w,
+               double eps) {
+  f32c(x, "x");
+  TORCH_CHECK(x.dim() == 2, "post_norm: x [T, W]");
+  auto rows = [&](const at::Tensor& t) {
+    TORCH_CHECK(t.is_cuda() && t.is_contiguous() && t.sizes() == x.sizes() &&
+                    t.scalar_type() == a.scalar_type(),
+                "post_norm: rows [T, W] of one activation dtype");
+  };
+  rows(a);
+  if (b) rows(*b);
+  if (h) rows(*h);
+  TORCH_CHECK(w.is_cuda() && w.is_contiguous() && w.numel() == x.size(1) &&
+                  w.scalar_type() == a.scalar_type(),
+              "post_norm: weight [W] of the activation dtype");
+  const at::DeviceGuard g(x.device());
+  rc_ok(mixk_post_norm(h ? h->data_ptr() : nullptr, x.data_ptr<float>(), static_cast<float>(alpha),
+                       a.data_ptr(), static_cast<float>(sa), b ? b->data_ptr() : nullptr,
+                       static_cast<float>(sb), w.data_ptr(), x.size(0), x.size(1),
+                       static_cast<float>(eps), code(a), cur_stream()),
+        "post_norm");
+}
+
 void proj_inv_rms(at::Tensor out, const at::Tensor& qx, const at::Tensor& kx, double eps) {
   f32c(out, "out");
   rows2d(qx, qx, "q");
@@ -804,12 +905,17 @@ TORCH_LIBRARY(atta_mix, m) {
   m.def("qk_norm_rope_cache(Tensor(a!) q_out, Tensor qx, Tensor kx, Tensor vx, Tensor? q_norm, "
         "Tensor? k_norm, float eps, Tensor positions, Tensor slot_mapping, Tensor cos_sin, "
         "Tensor(b!) k_cache, Tensor(c!) v_cache, bool rotate_half, bool norm_last, "
-        "Tensor? row_inv) -> ()");
-  m.def("rotary_table(Tensor(a!) out, Tensor positions, Tensor inv_freq) -> ()");
+        "Tensor? row_inv, float temp_coef, float temp_every, bool v_norm, Tensor? v_first, "
+        "float v_lambda, Tensor(d!)? v_out) -> ()");
+  m.def("rotary_table(Tensor(a!) out, Tensor positions, Tensor inv_freq, float mult) -> ()");
   m.def("sink_attention(Tensor(a!) out, Tensor q, Tensor k_cache, Tensor v_cache, "
         "Tensor block_tables, Tensor seq_kvlen, Tensor seq_qstart, Tensor tile_seq, "
         "Tensor tile_qoff, float scale, bool sink, int num_decode, int max_decode_kv, "
-        "Tensor? part, bool use_mfma, Tensor? sink_val, int window) -> ()");
+        "Tensor? part, bool use_mfma, Tensor? sink_val, int window, Tensor? gate) -> ()");
+  m.def("sigmoid_attention(Tensor(a!) out, Tensor q, Tensor k_cache, Tensor v_cache, "
+        "Tensor block_tables, Tensor seq_kvlen, Tensor seq_qstart, Tensor tile_seq, "
+        "Tensor tile_qoff, float scale, float cap, Tensor bias, Tensor talk, int num_decode, "
+        "int max_decode_kv, Tensor? part, bool use_mfma) -> ()");
   m.def("short_conv_silu(Tensor(a!) out, Tensor x, Tensor w, Tensor(b!) conv_state, "
         "Tensor positions, Tensor seq_qstart, Tensor seq_slot, Tensor? bias) -> ()");
   m.def("gated_delta_rule(Tensor(a!) out, Tensor qkv, Tensor beta, Tensor decay, Tensor a_log, "
@@ -823,7 +929,7 @@ TORCH_LIBRARY(atta_mix, m) {
   m.def("head_gate(Tensor(a!) out, Tensor o, Tensor gate) -> ()");
   m.def("latent_rope_cache(Tensor(a!) q_out, Tensor q_lat, Tensor qx, Tensor? kvx, Tensor? c_norm, "
         "float eps, Tensor slot_mapping, Tensor cos_sin, Tensor(b!) k_cache, Tensor(c!) v_cache, "
-        "Tensor(d!) c_out) -> ()");
+        "Tensor(d!) c_out, bool rotate_half) -> ()");
   m.def("gated_linear_scan(Tensor(a!) out, Tensor(b!) state, Tensor q, Tensor k, Tensor v, "
         "Tensor? dt, Tensor p0, Tensor p1, Tensor? p2, Tensor positions, Tensor seq_qstart, "
         "Tensor seq_slot, int H, int G, int dk, int dv, int mode) -> ()");
@@ -837,7 +943,7 @@ TORCH_LIBRARY(atta_mix, m) {
         "Tensor positions, Tensor seq_qstart, Tensor seq_slot) -> ()");
   m.def("pair_sum(Tensor(a!) out, Tensor y) -> ()");
   m.def("clamped_glu(Tensor(a!) out, Tensor gu, Tensor wts, float limit, float alpha) -> ()");
-  m.def("moe_route(Tensor(a!) idx, Tensor(b!) wts, Tensor logits, bool softmax, Tensor? correction, "
+  m.def("moe_route(Tensor(a!) idx, Tensor(b!) wts, Tensor logits, int score, Tensor? correction, "
         "int groups, int keep, bool renorm) -> ()");
   m.def("moe_experts(Tensor(a!) y, Tensor(b!) act, Tensor(c!) plan, Tensor h, Tensor idx, "
         "Tensor wts, Tensor w_gate, Tensor w_up, Tensor w_down, float limit, float alpha, "
@@ -846,6 +952,8 @@ TORCH_LIBRARY(atta_mix, m) {
         "int E, int split) -> ()");
   m.def("norm_add_norm(Tensor(a!)? h, Tensor(b!) x, Tensor? y, Tensor? w_post, Tensor? w_next, "
         "float eps, bool layer) -> ()");
+  m.def("post_norm(Tensor(a!)? h, Tensor(b!) x, float alpha, Tensor a, float sa, Tensor? b, "
+        "float sb, Tensor w, float eps) -> ()");
   m.def("proj_inv_rms(Tensor(a!) out, Tensor qx, Tensor kx, float eps) -> ()");
   m.def("scale_softcap(Tensor(a!) out, Tensor logits, float scale, float cap) -> ()");
 }
@@ -860,6 +968,7 @@ TORCH_LIBRARY_IMPL(atta_mix, CUDA, m) {
   m.impl("qk_norm_rope_cache", &qk_norm_rope_cache);
   m.impl("rotary_table", &rotary_table);
   m.impl("sink_attention", &sink_attention);
+  m.impl("sigmoid_attention", &sigmoid_attention);
   m.impl("short_conv_silu", &short_conv_silu);
   m.impl("gated_delta_rule", &gated_delta_rule);
   m.impl("embed_scale", &embed_scale);
@@ -880,6 +989,7 @@ TORCH_LIBRARY_IMPL(atta_mix, CUDA, m) {
   m.impl("moe_experts", &moe_experts);
   m.impl("moe_combine", &moe_combine);
   m.impl("norm_add_norm", &norm_add_norm);
+  m.impl("post_norm", &post_norm);
   m.impl("proj_inv_rms", &proj_inv_rms);
   m.impl("scale_softcap", &scale_softcap);
 }

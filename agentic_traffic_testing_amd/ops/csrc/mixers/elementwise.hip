@@ -355,13 +355,36 @@ __global__ void group_rms_norm_vec_kernel(T* __restrict__ out, const float* __re
 template <typename T>
 __global__ void head_gate_kernel(T* __restrict__ out, const T* __restrict__ o,
                                  const T* __restrict__ gate, int64_t gate_stride, int T_, int H,
-                                 int dv) {
+                                 int dv, int per_channel) {
   const int t = blockIdx.x;
   for (int i = threadIdx.x; i < H * dv; i += blockDim.x) {
     const int h = i / dv, j = i - h * dv;
-    const float gv = sigmoidf_(ldf(gate + t * gate_stride + h));
+    const float gv = sigmoidf_(ldf(gate + t * gate_stride + (per_channel ? i : h)));
     stf(out + static_cast<int64_t>(t) * H * dv + i,
         ldf(o + (static_cast<int64_t>(h) * T_ + t) * dv + j) * gv);
+  }
+}
+
+// dv % 8 == 0 and aligned rows: 8 channels per thread and round
+template <typename T>
+__global__ void head_gate_vec_kernel(T* __restrict__ out, const T* __restrict__ o,
+                                     const T* __restrict__ gate, int64_t gate_stride, int T_,
+                                     int H, int dv, int per_channel) {
+  const int t = blockIdx.x;
+  for (int i = threadIdx.x * 8; i < H * dv; i += blockDim.x * 8) {
+    const int h = i / dv, j = i - h * dv;
+    float v[8], g[8];
+    ld8(o + (static_cast<int64_t>(h) * T_ + t) * dv + j, v);
+    if (per_channel) {
+      ld8(gate + t * gate_stride + i, g);
+#pragma unroll
+      for (int e = 0; e < 8; ++e) v[e] *= sigmoidf_(g[e]);
+    } else {
+      const float gv = sigmoidf_(ldf(gate + t * gate_stride + h));
+#pragma unroll
+      for (int e = 0; e < 8; ++e) v[e] *= gv;
+    }
+    st8(out + static_cast<int64_t>(t) * H * dv + i, v);
   }
 }
 
@@ -526,10 +549,21 @@ extern "C" int mixk_group_rms_norm(void* out, const float* y, const void* gate,
 }
 
 extern "C" int mixk_head_gate(void* out, const void* o, const void* gate, int64_t gate_stride,
-                              int T_, int H, int dv, int dtype, hipStream_t st) {
+                              int T_, int H, int dv, int per_channel, int dtype, hipStream_t st) {
   if (T_ <= 0) return 0;
-  MIXK_DISPATCH(dtype, hipLaunchKernelGGL(head_gate_kernel<T>, dim3(T_), dim3(256), 0, st,
-                                          static_cast<T*>(out), static_cast<const T*>(o),
-                                          static_cast<const T*>(gate), gate_stride, T_, H, dv));
+  const uintptr_t mask = dtype == 2 ? 31 : 15;
+  const bool vec = dv % 8 == 0 && ((reinterpret_cast<uintptr_t>(out) | reinterpret_cast<uintptr_t>(o)) & mask) == 0 &&
+                   (!per_channel || ((reinterpret_cast<uintptr_t>(gate) & mask) == 0 && gate_stride % 8 == 0));
+#define MIXK_GATE(KERNEL)                                                                        \
+  hipLaunchKernelGGL(KERNEL<T>, dim3(T_), dim3(256), 0, st, static_cast<T*>(out),                \
+                     static_cast<const T*>(o), static_cast<const T*>(gate), gate_stride, T_, H,  \
+                     dv, per_channel)
+  MIXK_DISPATCH(dtype, {
+    if (vec)
+      MIXK_GATE(head_gate_vec_kernel);
+    else
+      MIXK_GATE(head_gate_kernel);
+  });
+#undef MIXK_GATE
   return static_cast<int>(hipGetLastError());
 }

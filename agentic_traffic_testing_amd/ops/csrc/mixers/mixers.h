@@ -27,16 +27,25 @@ int mixk_qk_norm_rope_cache(void* q_out, const void* qx, int64_t q_stride, const
                             const int* slot_mapping, const float* cos_sin, int n_freq,
                             void* k_cache, void* v_cache, int T, int H, int G, int dim, int vdim,
                             int block_size, int half, int norm_last, const float* row_inv,
-                            int dtype, hipStream_t st);
+                            float temp_coef, float temp_every, int v_norm, const void* v_first,
+                            float v_lambda, void* v_out, int dtype, hipStream_t st);
 int mixk_rotary_table(float* out, const int* positions, const float* inv_freq, int T, int n_freq,
-                      hipStream_t st);
+                      float mult, hipStream_t st);
 int mixk_sink_attention(void* out, const void* q, const void* k_cache, const void* v_cache,
                         const int* block_tables, int bt_width, const int* seq_kvlen,
                         const int* seq_qstart, const int* tile_seq, const int* tile_qoff,
                         int num_tiles, int num_decode, int max_decode_kv, float* part,
                         int max_parts, int H, int G, int dim, int vdim, int block_size,
-                        float scale, int sink, const float* sink_val, int window, int use_mfma,
-                        int dtype, hipStream_t st);
+                        float scale, int sink, const float* sink_val, int window,
+                        const void* gate, int64_t gate_stride, int use_mfma, int dtype,
+                        hipStream_t st);
+int mixk_sigmoid_attention(void* out, const void* q, const void* k_cache, const void* v_cache,
+                           const int* block_tables, int bt_width, const int* seq_kvlen,
+                           const int* seq_qstart, const int* tile_seq, const int* tile_qoff,
+                           int num_tiles, int num_decode, int max_decode_kv, float* part,
+                           int max_parts, int H, int G, int dim, int vdim, int block_size,
+                           float scale, float cap, const float* bias, const float* talk,
+                           int use_mfma, int dtype, hipStream_t st);
 int mixk_short_conv_silu(void* out, const void* x, int64_t x_stride, const void* w,
                          const void* bias, void* conv_state, const int* positions, const int* seq_qstart,
                          const int* seq_slot, int T, int S, int C, int taps, int dtype,
@@ -56,12 +65,13 @@ int mixk_group_rms_norm(void* out, const float* y, const void* gate, int64_t gat
                         const void* w, int T, int n_groups, int gs, float eps, int w_full,
                         int dtype, hipStream_t st);
 int mixk_head_gate(void* out, const void* o, const void* gate, int64_t gate_stride, int T, int H,
-                   int dv, int dtype, hipStream_t st);
-int mixk_latent_rope_cache(void* q_out, const void* q_lat, const void* qx, const void* kvx,
-                           int64_t kv_stride, const void* c_norm, float eps,
+                   int dv, int per_channel, int dtype, hipStream_t st);
+int mixk_latent_rope_cache(void* q_out, const void* q_lat, const void* qx, int64_t q_stride,
+                           const void* kvx, int64_t kv_stride, const void* c_norm, float eps,
                            const int* slot_mapping, const float* cos_sin, int n_freq,
                            void* k_cache, void* v_cache, void* c_out, int T, int H, int qdim,
-                           int rank, int rot, int block_size, int dtype, hipStream_t st);
+                           int rank, int rot, int block_size, int half, int dtype,
+                           hipStream_t st);
 int mixk_gated_linear_scan(float* out, float* state, const void* q, int64_t q_stride,
                            const void* k, int64_t k_stride, const void* v, int64_t v_stride,
                            const void* dt, int64_t dt_stride, const float* p0, const float* p1,
@@ -87,7 +97,7 @@ int mixk_clamped_glu(void* out, const void* gu, const float* wts, int R, int ff,
 int mixk_pair_sum(void* out, const void* y, int y_f32, int T, int top, int W, int dtype,
                   hipStream_t st);
 int mixk_moe_route(int* idx, float* wts, const float* logits, const float* correction, int T,
-                   int E, int top, int softmax, int groups, int keep, int renorm, hipStream_t st);
+                   int E, int top, int score, int groups, int keep, int renorm, hipStream_t st);
 int mixk_moe_experts(void* y, void* act, int* plan, const void* h, const int* idx,
                      const float* wts, const void* w_gate, const void* w_up, const void* w_down,
                      int T, int top, int E, int ff, int W, int64_t gu_estride, int max_tiles,
@@ -98,6 +108,8 @@ int mixk_moe_combine(void* out, const void* y, int y_f32, const int* idx, const 
                      int dtype, hipStream_t st);
 int mixk_norm_add_norm(void* h, float* x, const void* y, const void* w_post, const void* w_next,
                        int T, int W, float eps, int layer, int dtype, hipStream_t st);
+int mixk_post_norm(void* h, float* x, float alpha, const void* a, float sa, const void* b,
+                   float sb, const void* w, int T, int W, float eps, int dtype, hipStream_t st);
 int mixk_proj_inv_rms(float* out, const void* qx, int64_t q_stride, int nq, const void* kx,
                       int64_t k_stride, int nk, int T, float eps, int dtype, hipStream_t st);
 int mixk_scale_softcap(float* out, const void* x, int64_t n, float scale, float cap, int dtype,

@@ -3,8 +3,8 @@
 // expert into tiles, and grouped matrix products over the tiles - no host round trip, so a step
 // can be recorded in a graph.
 //
-// * moe_route: one wave per row of fp32 router logits [T, E]; scores = sigmoid, or softmax over
-//   the row; choice scores = scores (+ correction[e]); with groups > 1 a group (E / groups
+// * moe_route: one wave per row of fp32 router logits [T, E]; scores = sigmoid, softmax over
+//   the row, or the logits themselves (the weights are then their softmax over the chosen ones); choice scores = scores (+ correction[e]); with groups > 1 a group (E / groups
 //   neighbouring experts) scores its largest choice score, `keep` rounds of wave-wide arg-max
 //   pick the groups whose experts stay eligible; `top` rounds of wave-wide arg-max over the
 //   eligible choice scores (ties: lowest index) give idx [T, top]; wts [T, top] are the plain
@@ -44,6 +44,7 @@ namespace mixk {
 constexpr int kMoeRows = 64;        // rows per tile
 constexpr int kMoeFeat = 64;        // output features per workgroup
 constexpr int kMaxExperts = 1024;
+constexpr int kScoreSigmoid = 0, kScoreSoftmax = 1, kScoreLogit = 2;
 
 __device__ __forceinline__ void wave_argmax(float& best, int& be) {
 #pragma unroll
@@ -63,7 +64,7 @@ __device__ __forceinline__ void wave_argmax(float& best, int& be) {
 template <int PER>
 __global__ void __launch_bounds__(256)
 moe_route_kernel(int* __restrict__ idx, float* __restrict__ wts, const float* __restrict__ logits,
-                 const float* __restrict__ correction, int T_, int E, int top, int softmax,
+                 const float* __restrict__ correction, int T_, int E, int top, int score,
                  int groups, int keep, int renorm) {
   __shared__ float s_choice[4][PER * kWave];
   __shared__ unsigned char s_kept[4][PER * kWave];
@@ -82,7 +83,7 @@ moe_route_kernel(int* __restrict__ idx, float* __restrict__ wts, const float* __
     zmax = fmaxf(zmax, sc[j]);
     pick[j] = -1;
   }
-  if (softmax) {
+  if (score == kScoreSoftmax) {
 #pragma unroll
     for (int o = 32; o > 0; o >>= 1) zmax = fmaxf(zmax, __shfl_xor(zmax, o, kWave));
     float sum = 0.f;
@@ -94,7 +95,7 @@ moe_route_kernel(int* __restrict__ idx, float* __restrict__ wts, const float* __
     sum = wave_sum(sum);
 #pragma unroll
     for (int j = 0; j < PER; ++j) sc[j] = sc[j] / sum;
-  } else {
+  } else if (score == kScoreSigmoid) {
 #pragma unroll
     for (int j = 0; j < PER; ++j) sc[j] = sigmoidf_(sc[j]);
   }
@@ -168,17 +169,29 @@ moe_route_kernel(int* __restrict__ idx, float* __restrict__ wts, const float* __
         pick[j] = k;
       }
   }
+  if (score == kScoreLogit) {   // softmax over the chosen logits
+    float m = -INFINITY;
+#pragma unroll
+    for (int j = 0; j < PER; ++j)
+      if (pick[j] >= 0) m = fmaxf(m, sc[j]);
+#pragma unroll
+    for (int o = 32; o > 0; o >>= 1) m = fmaxf(m, __shfl_xor(m, o, kWave));
+#pragma unroll
+    for (int j = 0; j < PER; ++j)
+      if (pick[j] >= 0) sc[j] = expf(sc[j] - m);
+  }
   float tot = 0.f;
 #pragma unroll
   for (int j = 0; j < PER; ++j)
     if (pick[j] >= 0) tot += sc[j];
   tot = wave_sum(tot);
   if (!live) return;
+  const bool norm = renorm || score == kScoreLogit;
 #pragma unroll
   for (int j = 0; j < PER; ++j)
     if (pick[j] >= 0) {
       idx[static_cast<int64_t>(t) * top + pick[j]] = lane + j * kWave;
-      wts[static_cast<int64_t>(t) * top + pick[j]] = renorm ? sc[j] / (tot + 1e-20f) : sc[j];
+      wts[static_cast<int64_t>(t) * top + pick[j]] = norm ? sc[j] / (tot + 1e-20f) : sc[j];
     }
 }
 
@@ -621,15 +634,16 @@ extern "C" int mixk_clamped_glu(void* out, const void* gu, const float* wts, int
 }
 
 extern "C" int mixk_moe_route(int* idx, float* wts, const float* logits, const float* correction,
-                              int T_, int E, int top, int softmax, int groups, int keep,
+                              int T_, int E, int top, int score, int groups, int keep,
                               int renorm, hipStream_t st) {
   if (T_ <= 0) return 0;
+  if (score < kScoreSigmoid || score > kScoreLogit) return -1;
   if (E < 1 || E > kMaxExperts || top < 1 || top > E || groups < 1 || E % groups != 0 ||
       keep < 1 || keep > groups || top > keep * (E / groups))
     return -1;
 #define MIXK_ROUTE(PER)                                                                          \
   hipLaunchKernelGGL(moe_route_kernel<PER>, dim3((T_ + 3) / 4), dim3(256), 0, st, idx, wts,      \
-                     logits, correction, T_, E, top, softmax, groups, keep, renorm)
+                     logits, correction, T_, E, top, score, groups, keep, renorm)
   if (E <= kWave)
     MIXK_ROUTE(1);
   else if (E <= 4 * kWave)

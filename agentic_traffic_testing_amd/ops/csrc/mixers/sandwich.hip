@@ -1,6 +1,9 @@
-// Sandwich-norm layer boundary, the inverse RMS of whole q / k projections, and scaled,
-// soft-capped logits.
+// Sandwich-norm and post-norm layer boundaries, the inverse RMS of whole q / k projections, and
+// scaled, soft-capped logits.
 //
+// * post_norm: the residual itself is normed after the sum, one workgroup per row:
+//     x = rms(alpha x + sa a [+ sb b]) * w    (fp32, in place)
+//   and h, when given, takes the new x in the activation dtype - what the next sub-layer reads.
 // * norm_add_norm: one workgroup per row of the fp32 residual x [T, W]:
 //     x += norm(y) * w_post          (skipped when y is nullptr)
 //     h  = norm(x) * w_next          (skipped when h is nullptr)
@@ -136,6 +139,76 @@ __global__ void norm_add_norm_kernel(T* __restrict__ h, float* __restrict__ x,
 }
 
 template <typename T>
+__global__ void post_norm_vec_kernel(T* __restrict__ h, float* __restrict__ x, float alpha,
+                                     const T* __restrict__ a, float sa, const T* __restrict__ b,
+                                     float sb, const T* __restrict__ w, int W, float eps) {
+  __shared__ float scratch[16];
+  const int64_t base = static_cast<int64_t>(blockIdx.x) * W;
+  float xv[kSwGroups][8], av[kSwGroups][8];
+#pragma unroll
+  for (int g = 0; g < kSwGroups; ++g) {
+    const int i = (g * blockDim.x + threadIdx.x) * 8;
+    if (i < W) {
+      ld8(x + base + i, xv[g]);
+      ld8(a + base + i, av[g]);
+    }
+  }
+#pragma unroll
+  for (int g = 0; g < kSwGroups; ++g) {
+    const int i = (g * blockDim.x + threadIdx.x) * 8;
+    if (i < W) {
+      if (b != nullptr) {
+        float bv[8];
+        ld8(b + base + i, bv);
+#pragma unroll
+        for (int e = 0; e < 8; ++e) av[g][e] = sa * av[g][e] + sb * bv[e];
+      } else {
+#pragma unroll
+        for (int e = 0; e < 8; ++e) av[g][e] *= sa;
+      }
+#pragma unroll
+      for (int e = 0; e < 8; ++e) xv[g][e] = alpha * xv[g][e] + av[g][e];
+    }
+  }
+  float mean, inv;
+  row_stats<false>(xv, W, eps, scratch, mean, inv);
+#pragma unroll
+  for (int g = 0; g < kSwGroups; ++g) {
+    const int i = (g * blockDim.x + threadIdx.x) * 8;
+    if (i < W) {
+      float wv[8];
+      ld8(w + i, wv);
+#pragma unroll
+      for (int e = 0; e < 8; ++e) wv[e] = xv[g][e] * inv * wv[e];
+      st8(x + base + i, wv);
+      if (h != nullptr) st8(h + base + i, wv);
+    }
+  }
+}
+
+template <typename T>
+__global__ void post_norm_kernel(T* __restrict__ h, float* __restrict__ x, float alpha,
+                                 const T* __restrict__ a, float sa, const T* __restrict__ b,
+                                 float sb, const T* __restrict__ w, int W, float eps) {
+  __shared__ float scratch[16];
+  const int64_t base = static_cast<int64_t>(blockIdx.x) * W;
+  float ss = 0.f;
+  for (int i = threadIdx.x; i < W; i += blockDim.x) {
+    float y = sa * ldf(a + base + i);
+    if (b != nullptr) y += sb * ldf(b + base + i);
+    const float v = alpha * x[base + i] + y;
+    x[base + i] = v;   // re-read below by this thread only
+    ss += v * v;
+  }
+  const float inv = 1.0f / sqrtf(block_sum(ss, scratch) / static_cast<float>(W) + eps);
+  for (int i = threadIdx.x; i < W; i += blockDim.x) {
+    const float v = x[base + i] * inv * ldf(w + i);
+    x[base + i] = v;
+    if (h != nullptr) stf(h + base + i, v);
+  }
+}
+
+template <typename T>
 __global__ void proj_inv_rms_kernel(float* __restrict__ out, const T* __restrict__ qx,
                                     int64_t q_stride, int nq, const T* __restrict__ kx,
                                     int64_t k_stride, int nk, int T_, float eps, int vec) {
@@ -213,6 +286,27 @@ extern "C" int mixk_norm_add_norm(void* h, float* x, const void* y, const void* 
       MIXK_SANDWICH(norm_add_norm_kernel, false, 256);
   });
 #undef MIXK_SANDWICH
+  return static_cast<int>(hipGetLastError());
+}
+
+extern "C" int mixk_post_norm(void* h, float* x, float alpha, const void* a, float sa,
+                              const void* b, float sb, const void* w, int T_, int W, float eps,
+                              int dtype, hipStream_t st) {
+  if (T_ <= 0 || W <= 0) return 0;
+  int threads = sandwich_threads(W);
+  auto fits = [&](const void* p) { return p == nullptr || (dtype == 2 ? al32(p) : al16(p)); };
+  if (!(al32(x) && fits(h) && fits(a) && fits(b) && fits(w))) threads = 0;
+#define MIXK_POST(KERNEL, THREADS)                                                               \
+  hipLaunchKernelGGL(KERNEL<T>, dim3(T_), dim3(THREADS), 0, st, static_cast<T*>(h), x, alpha,    \
+                     static_cast<const T*>(a), sa, static_cast<const T*>(b), sb,                 \
+                     static_cast<const T*>(w), W, eps)
+  MIXK_DISPATCH(dtype, {
+    if (threads)
+      MIXK_POST(post_norm_vec_kernel, threads);
+    else
+      MIXK_POST(post_norm_kernel, 256);
+  });
+#undef MIXK_POST
   return static_cast<int>(hipGetLastError());
 }
 

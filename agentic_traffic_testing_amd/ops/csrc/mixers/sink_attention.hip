@@ -26,6 +26,9 @@
 // touch its edge; decode then runs only the partitions that overlap the window (partition
 // indices are relative to the first of them, for the partition kernel and the combine alike).
 //
+// A per-head output gate (`gate`) multiplies the result by sigmoid(gate[row, head]) in the kernel
+// that stores it.
+//
 // The sink enters as the initial state of the online softmax: running max = the sink's score,
 // running sum 1, zero accumulator.  The sink's score is 0, or one learned number per query head
 // (`sink_val`, unscaled).
@@ -51,7 +54,15 @@ struct AttnArgs {
   int bt_width, H, G, dim, vdim, block_size, sink, KT, max_parts, bs_shift;
   float scale;
   int window;   // 0: every earlier key
+  const void* gate;       // row-strided [T, H] of the activation dtype, or nullptr: head h's output
+  int64_t gate_stride;    // of row t is multiplied by sigmoid(gate[t, h])
 };
+
+template <typename T>
+__device__ __forceinline__ float head_gate_of(const AttnArgs& a, int64_t row, int head) {
+  if (a.gate == nullptr) return 1.0f;
+  return sigmoidf_(ldf(static_cast<const T*>(a.gate) + row * a.gate_stride + head));
+}
 
 // first key a query at position qpos sees
 __device__ __forceinline__ int window_start(int qpos, int window) {
@@ -204,7 +215,7 @@ sink_attention_rows_kernel(T* __restrict__ out, const T* __restrict__ q,
     }
     return;
   }
-  const float inv = l > 0.f ? 1.0f / l : 0.f;
+  const float inv = (l > 0.f ? 1.0f / l : 0.f) * head_gate_of<T>(a, row0 + qo + r, h0);
   T* o = out + (static_cast<int64_t>(row0 + qo + r) * H + h0) * vdim;
 #pragma unroll
   for (int j = 0; j < kMaxVPer; ++j) {
@@ -240,7 +251,7 @@ __global__ void sink_attention_combine_kernel(T* __restrict__ out, AttnArgs a) {
   }
   L = wave_sum(L) + (a.sink ? expf(sink_score - M) : 0.f);
   __syncthreads();
-  const float inv = L > 0.f ? 1.0f / L : 0.f;
+  const float inv = (L > 0.f ? 1.0f / L : 0.f) * head_gate_of<T>(a, a.seq_qstart[s], h);
   T* o = out + (static_cast<int64_t>(a.seq_qstart[s]) * a.H + h) * vdim;
   for (int d = lane; d < vdim; d += kWave) {
     float v = 0.f;
@@ -474,7 +485,7 @@ sink_attention_mfma_kernel(__bf16* __restrict__ out, const __bf16* __restrict__ 
     }
     return;
   }
-  const float inv = l > 0.f ? 1.0f / l : 0.f;
+  const float inv = (l > 0.f ? 1.0f / l : 0.f) * head_gate_of<__bf16>(a, qrow, head);
   __bf16* o = out + (qrow * H + head) * vdim;
 #pragma unroll
   for (int vt = 0; vt < NV; ++vt) {
@@ -573,15 +584,16 @@ extern "C" int mixk_sink_attention(void* out, const void* q, const void* k_cache
                                    const int* tile_seq, const int* tile_qoff, int num_tiles,
                                    int num_decode, int max_decode_kv, float* part, int max_parts,
                                    int H, int G, int dim, int vdim, int block_size, float scale,
-                                   int sink, const float* sink_val, int window, int use_mfma,
-                                   int dtype, hipStream_t st) {
+                                   int sink, const float* sink_val, int window,
+                                   const void* gate, int64_t gate_stride, int use_mfma, int dtype,
+                                   hipStream_t st) {
   if (num_tiles <= 0 && num_decode <= 0) return 0;
   if (vdim > 16 * kMaxVPer || G <= 0 || H % G != 0) return -1;
   int bs_shift = 0;
   while ((1 << bs_shift) < block_size) ++bs_shift;
   AttnArgs a{block_tables, seq_kvlen, seq_qstart, tile_seq, tile_qoff, part, sink ? sink_val : nullptr,
              bt_width, H, G, dim, vdim, block_size, sink, 0, max_parts, bs_shift, scale,
-             window > 0 ? window : 0};
+             window > 0 ? window : 0, gate, gate_stride};
   int rc = 0;
   if (use_mfma) {
     if (dtype != 0 || dim % 16 || vdim % 32 || dim > 256 || vdim > 256 || block_size < 8 ||

@@ -7,8 +7,10 @@ norms, sums and activations around them; hyper-connection streams, token shift, 
 recurrence, element-wise gates, GELU, and routed clamped-GLU or SiLU-GLU experts (grouped matrix
 products over rows sorted by expert; sigmoid or softmax routing, optionally with a choice
 correction and group-limited choice; identity experts), the sandwich-norm layer boundary (layer
-norm or RMS norm of a branch added to the fp32 residual, then the next norm), q / k norms over
-a whole projection, and scaled, soft-capped logits.
+norm or RMS norm of a branch added to the fp32 residual, then the next norm), the post-norm
+boundary (the residual itself normed after a weighted sum), q / k norms over a whole projection,
+values normed per head and mixed with an earlier layer's, a position-dependent query temperature,
+unnormalised sigmoid attention with head mixing, and scaled, soft-capped logits.
 
 Same device-strict dispatch as ``ops``: GPU tensors run the HIP kernels of
 ``ops/csrc/mixers`` (library ``_atta_mixers.so``, operators ``torch.ops.atta_mix.*``; built on
@@ -18,6 +20,7 @@ recurrent state, scores, norms, decays and gates are fp32 in both.
 """
 from __future__ import annotations
 
+import math
 import os
 from pathlib import Path
 
@@ -71,8 +74,10 @@ def _native():
 
 ATTN_TILE_TOKENS = 64     # query tokens per prefill attention tile (the block manager tiles by it)
 DECODE_PART_TOKENS = 128  # keys per decode-attention partition
+SIGMOID_PART_TOKENS = 64  # ... of the sigmoid attention
 ATTENTION_MFMA = os.environ.get("ATTA_MIX_ATTENTION_MFMA", "1") != "0"
 ACT_SILU, ACT_SIGMOID, ACT_GELU_TANH = 0, 1, 2
+_SCORE_CODES = {"sigmoid": 0, "softmax": 1, "logit": 2}
 _ACT_CODES = {"silu": ACT_SILU, "sigmoid": ACT_SIGMOID, "gelu_tanh": ACT_GELU_TANH}
 
 
@@ -100,6 +105,28 @@ def scaled_inv_freq(rot_dims: int, base: float, scaling, device) -> torch.Tensor
     return f.to(torch.float32).to(device)
 
 
+def yarn_inv_freq(rot_dims: int, base: float, scaling, device) -> tuple[torch.Tensor, float]:
+    """``inv_freq`` with YaRN scaling ``(factor, original, fast, slow)``, and the factor on cos and
+    sin, 0.1 ln(factor) + 1.  A pair index above ``lo`` starts to have its frequency divided by
+    ``factor``, one above ``hi`` has it divided fully, linearly in the index between them; lo and
+    hi are the indices whose pairs turn ``fast`` / ``slow`` times within ``original`` positions.
+    float64, rounded once to fp32."""
+    if scaling is None:
+        return inv_freq(rot_dims, base, device), 1.0
+    factor, original, fast, slow = (float(v) for v in scaling)
+
+    def index(turns):
+        return rot_dims * math.log(original / (turns * 2.0 * math.pi)) / (2.0 * math.log(base))
+
+    lo = max(math.floor(index(fast)), 0)
+    hi = min(math.ceil(index(slow)), rot_dims - 1)
+    i = torch.arange(rot_dims // 2, dtype=torch.float64)
+    f = torch.pow(torch.tensor(float(base), dtype=torch.float64), -2.0 * i / rot_dims)
+    ramp = ((i - lo) / max(hi - lo, 0.001)).clamp(0.0, 1.0)
+    f = f / factor * ramp + f * (1.0 - ramp)
+    return f.to(torch.float32).to(device), 0.1 * math.log(factor) + 1.0
+
+
 def embed_pair(table, pair_table, ids, positions, seq_qstart, seq_slot, prev_token, mul_prev,
                mul_cur, buckets):
     if not table.is_cuda:
@@ -119,30 +146,39 @@ def rms_norm_f32(x, w, eps, one_plus=True, dtype=torch.bfloat16, out=None):
     return out
 
 
-def rotary_table(positions, inv_freq_t):
-    """fp32 [T, 2 n]: cos | sin of position * inv_freq[i]; one per step and rotary setting,
-    shared by every layer that uses it."""
+def rotary_table(positions, inv_freq_t, mult=1.0):
+    """fp32 [T, 2 n]: cos | sin of position * inv_freq[i], both times ``mult``; one per step and
+    rotary setting, shared by every layer that uses it."""
     if not positions.is_cuda:
-        return mref.rotary_table(positions, inv_freq_t)
+        return mref.rotary_table(positions, inv_freq_t, mult)
     out = torch.empty(positions.shape[0], 2 * inv_freq_t.shape[0], dtype=torch.float32,
                       device=positions.device)
-    _native().rotary_table(out, positions, inv_freq_t)
+    _native().rotary_table(out, positions, inv_freq_t, float(mult))
     return out
 
 
 def qk_norm_rope_cache(qx, kx, vx, q_norm, k_norm, eps, positions, slot_mapping, cos_sin,
                        k_cache, v_cache, heads, kv_heads, dim, vdim, rotate_half_pairs=False,
-                       norm_last=False, whole_norm=False):
+                       norm_last=False, whole_norm=False, q_temp=None, v_norm=False, v_first=None,
+                       v_lambda=0.0, v_out=None):
     """qx / kx / vx: row-strided [T, heads * dim] / [T, kv_heads * dim] / [T, kv_heads * vdim];
     cos_sin: ``rotary_table`` of the step's positions.  ``q_norm`` / ``k_norm`` None: the norm
     has no weight; ``rotate_half_pairs``: channel i pairs with i + n_freq instead of
     (2i, 2i + 1); ``norm_last``: rotate first, then norm; ``whole_norm``: q (and k) are normed
     over the whole projection, all heads at once, with weights [heads * dim] ([kv_heads * dim]) -
-    a one-wave-per-row kernel computes the two inverse root mean squares of every row first."""
+    a one-wave-per-row kernel computes the two inverse root mean squares of every row first;
+    ``q_temp`` (coef, every): q is multiplied by 1 + coef ln(floor((position + 1) / every) + 1).
+    Values: ``v_norm`` divides every head's value by its root mean square over vdim (no weight),
+    ``v_first`` [T, kv_heads * vdim] then mixes them, (1 - v_lambda) v + v_lambda v_first; what
+    results is cached, and stored to ``v_out`` [T, kv_heads * vdim] when given (rows without a
+    cache slot excepted)."""
+    if q_temp is not None and norm_last:
+        raise ValueError("a query temperature goes with the norm before the rotation")
     if not qx.is_cuda:
         return mref.qk_norm_rope_cache(qx, kx, vx, q_norm, k_norm, eps, positions, slot_mapping,
                                        cos_sin, k_cache, v_cache, heads, kv_heads, dim, vdim,
-                                       rotate_half_pairs, norm_last, whole_norm)
+                                       rotate_half_pairs, norm_last, whole_norm, q_temp, v_norm,
+                                       v_first, v_lambda, v_out)
     if whole_norm and norm_last:
         raise ValueError("a norm over the whole projection precedes the rotation")
     q = torch.empty(qx.shape[0], heads, dim, dtype=qx.dtype, device=qx.device)
@@ -151,7 +187,10 @@ def qk_norm_rope_cache(qx, kx, vx, q_norm, k_norm, eps, positions, slot_mapping,
         row_inv = torch.empty(qx.shape[0], 2, dtype=torch.float32, device=qx.device)
         _native().proj_inv_rms(row_inv, qx, kx, eps)
     _native().qk_norm_rope_cache(q, qx, kx, vx, q_norm, k_norm, eps, positions, slot_mapping,
-                                 cos_sin, k_cache, v_cache, rotate_half_pairs, norm_last, row_inv)
+                                 cos_sin, k_cache, v_cache, rotate_half_pairs, norm_last, row_inv,
+                                 float(q_temp[0]) if q_temp else 0.0,
+                                 float(q_temp[1]) if q_temp else 1.0, bool(v_norm), v_first,
+                                 float(v_lambda), v_out)
     return q
 
 
@@ -163,7 +202,8 @@ def mfma_attention_ok(q, k_cache, v_cache) -> bool:
 
 
 def sink_attention(q, k_cache, v_cache, block_tables, seq_kvlen, seq_qstart, tile_seq, tile_qoff,
-                   scale, sink=True, num_decode=0, max_decode_kv=0, sink_values=None, window=0):
+                   scale, sink=True, num_decode=0, max_decode_kv=0, sink_values=None, window=0,
+                   gate=None):
     """Causal attention of every portion's rows over its sequence's pages
     (k_cache [nb, G, BS, d], v_cache [nb, G, dv, BS]).  Sequences [0, num_decode) have one
     query row each and go through the partitioned decode kernel (``max_decode_kv``: their
@@ -171,11 +211,12 @@ def sink_attention(q, k_cache, v_cache, block_tables, seq_kvlen, seq_qstart, til
     ATTN_TILE_TOKENS query rows of every other portion (sequence index, row offset in it).
     ``sink_values``: fp32 [H], the sink's (unscaled) score per query head instead of 0.
     ``window`` > 0: a row at position i sees keys j with 0 <= i - j < window (decode then runs
-    only the partitions that overlap the window)."""
+    only the partitions that overlap the window).
+    ``gate`` [T, H] (row-strided): head h's output of row t is multiplied by sigmoid(gate[t, h])."""
     window = int(window)
     if not q.is_cuda:
         return mref.sink_attention(q, k_cache, v_cache, block_tables, seq_kvlen, seq_qstart,
-                                   scale, sink, sink_values, window)
+                                   scale, sink, sink_values, window, gate)
     out = torch.empty(q.shape[0], q.shape[1], v_cache.shape[2], dtype=q.dtype, device=q.device)
     part = None
     if num_decode > 0:
@@ -188,7 +229,30 @@ def sink_attention(q, k_cache, v_cache, block_tables, seq_kvlen, seq_qstart, til
         _native().sink_attention(out, q, k_cache, v_cache, block_tables, seq_kvlen, seq_qstart,
                                  tile_seq, tile_qoff, scale, sink, num_decode,
                                  max(1, int(max_decode_kv)), part,
-                                 mfma_attention_ok(q, k_cache, v_cache), sink_values, window)
+                                 mfma_attention_ok(q, k_cache, v_cache), sink_values, window, gate)
+    return out
+
+
+def sigmoid_attention(q, k_cache, v_cache, block_tables, seq_kvlen, seq_qstart, tile_seq,
+                      tile_qoff, scale, softcap, bias, talk, num_decode=0, max_decode_kv=0):
+    """Causal attention without a softmax, over the same pages and batch layout as
+    ``sink_attention``: head g gives key j the weight w_g = sigmoid(c tanh(scale q_g.k / c) +
+    bias[g]) (``softcap`` c; 0: sigmoid(scale q_g.k + bias[g])), not normalised over the keys, and
+    head h sums its KV head's values with the mixed weights sum_g talk[h, g] w_g.  bias fp32 [H],
+    talk fp32 [H, H] (values a bf16 checkpoint holds: the bf16 kernel reads them as bf16)."""
+    if not q.is_cuda:
+        return mref.sigmoid_attention(q, k_cache, v_cache, block_tables, seq_kvlen, seq_qstart,
+                                      scale, float(softcap), bias, talk)
+    out = torch.empty(q.shape[0], q.shape[1], v_cache.shape[2], dtype=q.dtype, device=q.device)
+    part = None
+    if num_decode > 0:
+        parts = max(1, -(-int(max_decode_kv) // SIGMOID_PART_TOKENS))
+        part = torch.empty(num_decode, q.shape[1], parts, v_cache.shape[2], dtype=torch.float32,
+                           device=q.device)
+    if tile_seq.shape[0] > 0 or num_decode > 0:
+        _native().sigmoid_attention(out, q, k_cache, v_cache, block_tables, seq_kvlen, seq_qstart,
+                                    tile_seq, tile_qoff, float(scale), float(softcap), bias, talk,
+                                    num_decode, max(1, int(max_decode_kv)), part, ATTENTION_MFMA)
     return out
 
 
@@ -291,7 +355,8 @@ def group_rms_norm(y, gate, w, n_groups, eps, dtype=torch.bfloat16):
 
 
 def head_gate(o, gate):
-    """o [H, T, dv] (head-major) times sigmoid(gate [T, H]) -> [T, H * dv]."""
+    """o [H, T, dv] (head-major) times sigmoid(gate) -> [T, H * dv]; gate [T, H] (one number per
+    head) or [T, H * dv] (one per channel)."""
     if not o.is_cuda:
         return mref.head_gate(o, gate)
     H, T, dv = o.shape
@@ -300,23 +365,25 @@ def head_gate(o, gate):
     return out
 
 
-def latent_rope_cache(q_lat, qx, kvx, c_norm, eps, slot_mapping, cos_sin, k_cache, v_cache):
+def latent_rope_cache(q_lat, qx, kvx, c_norm, eps, slot_mapping, cos_sin, k_cache, v_cache,
+                      rotate_half_pairs=True):
     """Front end of latent attention over one shared compressed K / V head.  q_lat [H, T, rank]:
-    queries times the key up-projection; qx [T, H, qdim + rot]: its last ``rot`` channels are
-    rotated (rotate-half pairs, table ``cos_sin``); returns the absorbed queries
+    queries times the key up-projection; qx [T, H, qdim + rot] (row-strided): its last ``rot``
+    channels are rotated (pairs (i, i + n_freq), or (2i, 2i + 1) without ``rotate_half_pairs``;
+    table ``cos_sin``); returns the absorbed queries
     [T, H, rank + rot].  kvx [T, rank + rot] (or None for a layer that reads another layer's
     pages): the first ``rank`` channels are RMS-normed with weight ``c_norm``, the rest rotated;
     [latent | rotated key] goes to k_cache [nb, 1, BS, rank + rot], the latent to the
     channel-major v_cache [nb, 1, rank, BS]."""
     if not qx.is_cuda:
         return mref.latent_rope_cache(q_lat, qx, kvx, c_norm, eps, slot_mapping, cos_sin, k_cache,
-                                      v_cache)
+                                      v_cache, rotate_half_pairs)
     H, T, rank = q_lat.shape
     rot = k_cache.shape[3] - rank
     q = torch.empty(T, H, rank + rot, dtype=qx.dtype, device=qx.device)
     c_out = torch.empty(T if kvx is not None else 0, rank, dtype=qx.dtype, device=qx.device)
     _native().latent_rope_cache(q, q_lat, qx, kvx, c_norm, eps, slot_mapping, cos_sin, k_cache,
-                                v_cache, c_out)
+                                v_cache, c_out, rotate_half_pairs)
     return q
 
 
@@ -482,20 +549,21 @@ def _moe_experts_library(h, idx, wts, w_gu, w_down, limit, alpha, silu_glu=False
 
 def moe_route(logits, top, score="sigmoid", correction=None, groups=1, keep=1, renorm=False):
     """fp32 router logits [T, E] -> (expert index int32 [T, top], score fp32 [T, top]) of every
-    row's ``top`` largest scores (ties: lowest index).  ``score``: "sigmoid", or "softmax" over
-    the row.  ``correction`` fp32 [E] is added to the scores for the choice only (the returned
+    row's ``top`` largest scores (ties: lowest index).  ``score``: "sigmoid", "softmax" over
+    the row, or "logit" (the logits choose, the weights are their softmax over the chosen ones).  ``correction`` fp32 [E] is added to the scores for the choice only (the returned
     weights are the plain scores).  ``groups`` > 1: the experts form that many equal runs of
     neighbours, a group's score is its largest choice score, and only experts of the ``keep``
     best groups can be chosen.  ``renorm``: the chosen scores are divided by their sum + 1e-20."""
     E = logits.shape[1]
+    code = _SCORE_CODES[score]
     if groups < 1 or E % groups or not 1 <= keep <= groups or top > keep * (E // groups):
         raise ValueError("moe_route: groups must split the experts evenly and hold `top` of them")
     if not logits.is_cuda:
-        return mref.moe_route(logits, top, score == "softmax", correction, groups, keep, renorm)
+        return mref.moe_route(logits, top, score, correction, groups, keep, renorm)
     T = logits.shape[0]
     idx = torch.empty(T, top, dtype=torch.int32, device=logits.device)
     wts = torch.empty(T, top, dtype=torch.float32, device=logits.device)
-    _native().moe_route(idx, wts, logits, score == "softmax", correction, groups, keep, renorm)
+    _native().moe_route(idx, wts, logits, code, correction, groups, keep, renorm)
     return idx, wts
 
 
@@ -558,6 +626,17 @@ def norm_add_norm(x, y, w_post, w_next, eps, kind="layer", dtype=torch.bfloat16)
     h = torch.empty(x.shape, dtype=dtype, device=x.device) if w_next is not None else None
     _native().norm_add_norm(h, x, y, w_post, w_next, eps, kind == "layer")
     return h
+
+
+def post_norm(x, alpha, a, sa, b, sb, w, eps, dtype=torch.bfloat16):
+    """Layer boundary of a post-norm residual in one pass: x (fp32 [T, W], in place) =
+    rms(alpha x + sa a [+ sb b]) * w; returns x as the next sub-layer reads it, in ``dtype``
+    (x itself for fp32)."""
+    if not x.is_cuda:
+        return mref.post_norm(x, alpha, a, sa, b, sb, w, eps, dtype)
+    h = torch.empty(x.shape, dtype=dtype, device=x.device) if dtype != torch.float32 else None
+    _native().post_norm(h, x, float(alpha), a, float(sa), b, float(sb), w, eps)
+    return x if h is None else h
 
 
 def scale_softcap(logits, scale=1.0, cap=0.0):

@@ -47,10 +47,10 @@ def rms_norm_f32(x, w, eps, one_plus, dtype):
     return (xf * torch.rsqrt(xf.pow(2).mean(-1, keepdim=True) + eps) * g).to(dtype)
 
 
-def rotary_table(positions, inv_freq):
-    """fp32 [T, 2 n]: cos | sin of position * inv_freq[i] (fp32 angles)."""
+def rotary_table(positions, inv_freq, mult=1.0):
+    """fp32 [T, 2 n]: cos | sin of position * inv_freq[i] (fp32 angles), times ``mult``."""
     ang = positions.float()[:, None] * inv_freq.float()[None, :]
-    return torch.cat([torch.cos(ang), torch.sin(ang)], 1)
+    return torch.cat([torch.cos(ang), torch.sin(ang)], 1) * mult
 
 
 def rotate_interleaved(x, cos_sin):
@@ -67,19 +67,30 @@ def rotate_interleaved(x, cos_sin):
 
 def qk_norm_rope_cache(qx, kx, vx, q_norm, k_norm, eps, positions, slot_mapping, cos_sin,
                        k_cache, v_cache, heads, kv_heads, dim, vdim, rotate_half_pairs=False,
-                       norm_last=False, whole_norm=False):
+                       norm_last=False, whole_norm=False, q_temp=None, v_norm=False, v_first=None,
+                       v_lambda=0.0, v_out=None):
     """Per-head RMS norm (plain weight, or none when ``q_norm`` / ``k_norm`` is None; with
     ``whole_norm`` one norm over all heads of the projection with weights [heads * dim]) and rotary
     positions on q [T, heads * dim] and k [T, kv_heads * dim] (row-strided views); returns
     q [T, heads, dim] and writes k and v [T, kv_heads * vdim] into the paged caches
     k_cache [nb, kv_heads, BS, dim], v_cache [nb, kv_heads, vdim, BS] (channel-major pages).
     ``rotate_half_pairs``: channel i pairs with i + n instead of (2i, 2i + 1); ``norm_last``: the
-    norm follows the rotation instead of preceding it."""
+    norm follows the rotation instead of preceding it; ``q_temp`` (coef, every): q times
+    1 + coef ln(floor((position + 1) / every) + 1).  ``v_norm``: a head's value is divided by its
+    root mean square; ``v_first`` [T, kv_heads * vdim]: then (1 - v_lambda) v + v_lambda v_first;
+    ``v_out`` takes the cached values."""
     T = qx.shape[0]
     dt = qx.dtype
     q = qx.reshape(T, heads, dim).float()
     k = kx.reshape(T, kv_heads, dim).float()
-    v = vx.reshape(T, kv_heads, vdim)
+    v = vx.reshape(T, kv_heads, vdim).float()
+    if v_norm:
+        v = v * torch.rsqrt(v.pow(2).mean(-1, keepdim=True) + eps)
+    if v_first is not None:
+        v = (1.0 - v_lambda) * v + v_lambda * v_first.float().view(T, kv_heads, vdim)
+    v = v.to(dt)
+    if v_out is not None:
+        v_out.copy_(v.reshape(T, kv_heads * vdim))
 
     def nrm(x, w):
         if whole_norm:
@@ -92,7 +103,11 @@ def qk_norm_rope_cache(qx, kx, vx, q_norm, k_norm, eps, positions, slot_mapping,
     if norm_last:
         q, k = nrm(rot(q, cos_sin), q_norm).to(dt), nrm(rot(k, cos_sin), k_norm).to(dt)
     else:
-        q, k = rot(nrm(q, q_norm), cos_sin).to(dt), rot(nrm(k, k_norm), cos_sin).to(dt)
+        q, k = rot(nrm(q, q_norm), cos_sin), rot(nrm(k, k_norm), cos_sin).to(dt)
+        if q_temp is not None:
+            step = torch.floor((positions[:T].float() + 1.0) / q_temp[1])
+            q = q * (1.0 + q_temp[0] * torch.log(step + 1.0))[:, None, None]
+        q = q.to(dt)
     bs = k_cache.shape[2]
     sm = slot_mapping.long()
     ok = sm >= 0
@@ -104,11 +119,12 @@ def qk_norm_rope_cache(qx, kx, vx, q_norm, k_norm, eps, positions, slot_mapping,
 
 
 def sink_attention(q, k_cache, v_cache, block_tables, seq_kvlen, seq_qstart, scale, sink,
-                   sink_values=None, window=0):
+                   sink_values=None, window=0, gate=None):
     """Causal paged attention of every portion's rows over its sequence's cached keys; fp32
     scores and weights; ``sink`` adds exp(s - max) to each denominator, s = 0 or the head's
     entry of ``sink_values`` [H]; ``window`` > 0: a row at position i sees keys j with
-    0 <= i - j < window.  q [T, H, d] -> [T, H, dv]."""
+    0 <= i - j < window; ``gate`` [T, H]: outputs times sigmoid(gate).  q [T, H, d] ->
+    [T, H, dv]."""
     T, H, _ = q.shape
     G, bs, dv = k_cache.shape[1], k_cache.shape[2], v_cache.shape[2]
     out = torch.zeros(T, H, dv, dtype=q.dtype, device=q.device)
@@ -140,7 +156,40 @@ def sink_attention(q, k_cache, v_cache, block_tables, seq_kvlen, seq_qstart, sca
         den = e.sum(-1, keepdim=True)
         if sink:
             den = den + torch.exp(sv - m)
-        out[a:b] = torch.einsum("hqk,hkd->qhd", e / den, v).to(q.dtype)
+        o = torch.einsum("hqk,hkd->qhd", e / den, v)
+        if gate is not None:
+            o = o * torch.sigmoid(gate[a:b].float())[:, :, None]
+        out[a:b] = o.to(q.dtype)
+    return out
+
+
+def sigmoid_attention(q, k_cache, v_cache, block_tables, seq_kvlen, seq_qstart, scale, softcap,
+                      bias, talk):
+    """Causal paged attention with unnormalised weights sigmoid(c tanh(scale q.k / c) + bias[h])
+    (c = ``softcap``; 0: none), mixed over the heads by talk [H, H] before the values are summed;
+    fp32 scores, weights and mix.  q [T, H, d] -> [T, H, dv]."""
+    T, H, _ = q.shape
+    G, bs, dv = k_cache.shape[1], k_cache.shape[2], v_cache.shape[2]
+    out = torch.zeros(T, H, dv, dtype=q.dtype, device=q.device)
+    qs = seq_qstart.tolist()
+    for s, kvlen in enumerate(seq_kvlen.tolist()):
+        a, b = qs[s], qs[s + 1]
+        if kvlen <= 0 or b <= a:
+            continue
+        nblk = (kvlen + bs - 1) // bs
+        pages = block_tables[s, :nblk].long()
+        k = k_cache[pages].permute(1, 0, 2, 3).reshape(G, nblk * bs, -1)[:, :kvlen].float()
+        v = v_cache[pages].permute(1, 0, 3, 2).reshape(G, nblk * bs, dv)[:, :kvlen].float()
+        k, v = k.repeat_interleave(H // G, 0), v.repeat_interleave(H // G, 0)
+        sc = torch.einsum("qhd,hkd->hqk", q[a:b].float(), k) * scale
+        if softcap > 0:
+            sc = softcap * torch.tanh(sc / softcap)
+        w = torch.sigmoid(sc + bias.float()[:, None, None])
+        qpos = torch.arange(kvlen - (b - a), kvlen, device=q.device)
+        kpos = torch.arange(kvlen, device=q.device)
+        w = w.masked_fill(kpos[None, None, :] > qpos[None, :, None], 0.0)
+        w = torch.einsum("hg,gqk->hqk", talk.float(), w)
+        out[a:b] = torch.einsum("hqk,hkd->qhd", w, v).to(q.dtype)
     return out
 
 
@@ -267,8 +316,9 @@ def group_rms_norm(y, gate, w, n_groups, eps, dtype):
 
 def head_gate(o, gate):
     H, T, dv = o.shape
-    g = torch.sigmoid(gate.float())                       # [T, H]
-    return (o.float().permute(1, 0, 2) * g[:, :, None]).to(o.dtype).reshape(T, H * dv)
+    g = torch.sigmoid(gate.float())                       # [T, H] or [T, H * dv]
+    g = g[:, :, None] if g.shape[1] == H else g.reshape(T, H, dv)
+    return (o.float().permute(1, 0, 2) * g).to(o.dtype).reshape(T, H * dv)
 
 
 def rotate_half(x, cos_sin):
@@ -281,17 +331,19 @@ def rotate_half(x, cos_sin):
     return torch.cat([u * c - v * s, v * c + u * s, x[..., 2 * n:]], -1)
 
 
-def latent_rope_cache(q_lat, qx, kvx, c_norm, eps, slot_mapping, cos_sin, k_cache, v_cache):
+def latent_rope_cache(q_lat, qx, kvx, c_norm, eps, slot_mapping, cos_sin, k_cache, v_cache,
+                      rotate_half_pairs=True):
     H, T, rank = q_lat.shape
     rot = k_cache.shape[3] - rank
     dt = qx.dtype
-    qr = rotate_half(qx[..., qx.shape[2] - rot:].float(), cos_sin).to(dt)
+    turn = rotate_half if rotate_half_pairs else rotate_interleaved
+    qr = turn(qx[..., qx.shape[2] - rot:].float(), cos_sin).to(dt)
     q = torch.cat([q_lat.permute(1, 0, 2), qr], -1).contiguous()
     if kvx is not None:
         kv = kvx.float()
         c = kv[:, :rank]
         c = (c * torch.rsqrt(c.pow(2).mean(-1, keepdim=True) + eps) * c_norm.float()).to(dt)
-        kr = rotate_half(kv[:, rank:], cos_sin).to(dt)
+        kr = turn(kv[:, None, rank:], cos_sin)[:, 0].to(dt)
         bs = k_cache.shape[2]
         sm = slot_mapping.long()
         ok = sm >= 0
@@ -413,14 +465,15 @@ def gelu(x, tanh_form=False):
     return F.gelu(x.float(), approximate="tanh" if tanh_form else "none").to(x.dtype)
 
 
-def moe_route(logits, top, softmax=False, correction=None, groups=1, keep=1, renorm=False):
-    """Scores (sigmoid, or softmax over the row) of fp32 router logits [T, E]; the ``top`` largest
+def moe_route(logits, top, score="sigmoid", correction=None, groups=1, keep=1, renorm=False):
+    """Scores (sigmoid, softmax over the row, or the logits themselves) of fp32 router logits [T, E]; the ``top`` largest
     per row (ties: lowest index) -> (int32 [T, top], fp32 [T, top]).  ``correction`` [E] is added
     to the scores for the choice only; with ``groups`` > 1 only experts of the ``keep`` groups (equal
     runs of neighbours) with the largest best choice score can be chosen; ``renorm``: the chosen
-    scores are divided by their sum + 1e-20."""
+    scores are divided by their sum + 1e-20; "logit" scores give the softmax over the chosen."""
     z = logits.float()
-    s = torch.softmax(z, 1) if softmax else torch.sigmoid(z)
+    s = {"softmax": lambda: torch.softmax(z, 1), "sigmoid": lambda: torch.sigmoid(z),
+         "logit": lambda: z}[score]()
     c = s + correction.float() if correction is not None else s.clone()
     T, E = s.shape
     if groups > 1:
@@ -431,7 +484,9 @@ def moe_route(logits, top, softmax=False, correction=None, groups=1, keep=1, ren
         c = c.masked_fill(~allow.repeat_interleave(E // groups, 1), float("-inf"))
     order = torch.argsort(c, dim=1, descending=True, stable=True)[:, :top]
     w = torch.gather(s, 1, order)
-    if renorm:
+    if score == "logit":
+        w = torch.softmax(w, 1)
+    elif renorm:
         w = w / (w.sum(1, keepdim=True) + 1e-20)
     return order.to(torch.int32), w
 
@@ -493,6 +548,16 @@ def norm_add_norm(x, y, w_post, w_next, eps, layer, dtype):
     if y is not None:
         x += nrm(y, w_post)
     return nrm(x, w_next).to(dtype) if w_next is not None else None
+
+
+def post_norm(x, alpha, a, sa, b, sb, w, eps, dtype):
+    """x (fp32 [T, W], in place) = v / sqrt(mean(v^2) + eps) * w of v = alpha x + sa a [+ sb b];
+    returns x in ``dtype``."""
+    v = alpha * x + sa * a.float()
+    if b is not None:
+        v = v + sb * b.float()
+    x.copy_(v * torch.rsqrt(v.pow(2).mean(-1, keepdim=True) + eps) * w.float())
+    return x if dtype == torch.float32 else x.to(dtype)
 
 
 def scale_softcap(logits, scale, cap):

@@ -678,7 +678,8 @@ def test_moe_route_grouped(E, top, groups, keep, softmax):
             for renorm in (True, False):
                 idx, wts = mx.moe_route(logits.cuda(), top, "softmax" if softmax else "sigmoid",
                                         None if c is None else c.cuda(), groups, keep, renorm)
-                ri, rw = mref.moe_route(logits, top, softmax, c, groups, keep, renorm)
+                ri, rw = mref.moe_route(logits, top, "softmax" if softmax else "sigmoid", c, groups,
+                                            keep, renorm)
                 # the order among the chosen is by choice score; compare as sets with weights
                 so, ro = torch.argsort(idx.cpu(), 1), torch.argsort(ri, 1)
                 same = (torch.gather(idx.cpu(), 1, so) == torch.gather(ri, 1, ro)).all(1)
@@ -700,7 +701,7 @@ def test_moe_experts_silu_identity(dt, T, E, ident, top, ff, W):
     h = torch.randn(T, W).to(dt)
     wgu = (torch.randn(E, 2 * ff, W) * 2 / W ** 0.5).to(dt)
     wd = (torch.randn(E, W, ff) / ff ** 0.5).to(dt)
-    idx, wts = mref.moe_route(torch.randn(T, E + ident) * 2, top, True, None, 1, 1, True)
+    idx, wts = mref.moe_route(torch.randn(T, E + ident) * 2, top, "softmax", None, 1, 1, True)
     add = torch.randn(T, W).to(dt)
     t = dict(atol=6e-2, rtol=3e-2) if dt == torch.bfloat16 else dict(atol=5e-5, rtol=5e-5)
     for addend in (add, None):
