@@ -730,3 +730,151 @@ def test_strided_glu_and_softcap(dt):
         got = mx.scale_softcap(z.cuda(), scale, cap)
         assert got.dtype == torch.float32
         assert torch.allclose(got.cpu(), mref.scale_softcap(z, scale, cap), atol=2e-5, rtol=1e-5)
+
+
+# ---- sigmoid attention, post-norm boundary, value path, gates ------------------------------------
+
+def ragged_pages(md, G, dim, vdim, bs, dt, seed=0):
+    g = torch.Generator().manual_seed(seed)
+    nb = md["num_pages"]
+    return (torch.randn(nb, G, bs, dim, generator=g).to(dt),
+            torch.randn(nb, G, vdim, bs, generator=g).to(dt))
+
+
+@pytest.mark.parametrize("dt", DTYPES)
+@pytest.mark.parametrize("H,G,dim,vdim,bs,cap", [
+    (6, 6, 40, 48, 16, 7.0), (8, 2, 64, 64, 16, 0.0), (12, 4, 128, 128, 32, 20.0),
+    (24, 8, 128, 96, 8, 15.0), (32, 8, 128, 128, 16, 30.0), (3, 1, 16, 16, 16, 5.0),
+    (20, 2, 72, 32, 16, 9.0), (5, 5, 13, 9, 16, 4.0), (40, 8, 32, 16, 16, 6.0),
+    (4, 2, 32, 32, 12, 6.0), (8, 8, 192, 160, 16, 11.0), (1, 1, 8, 16, 16, 0.0)])
+def test_sigmoid_attention(dt, H, G, dim, vdim, bs, cap):
+    torch.manual_seed(1)
+    lens, starts = [1, 1, 37, 2, 150, 64, 16], [0, 170, 0, 131, 45, 200, 15]
+    md = ragged(lens, starts, list(range(7)), bs=bs, width=48)
+    T = int(md["seq_qstart"][-1])
+    q = torch.randn(T, H, dim).to(dt)
+    kc, vc = ragged_pages(md, G, dim, vdim, bs, dt)
+    bias = torch.randn(H) - 3.0
+    talk = (torch.eye(H) + 0.3 * torch.randn(H, H)).to(torch.bfloat16).float()
+    scale = 1.7 * dim ** -0.5
+    want = mref.sigmoid_attention(q, kc, vc, md["block_tables"], md["seq_kvlen"],
+                                  md["seq_qstart"], scale, cap, bias, talk).float()
+    g = cuda(md)
+    for nd in (0, 2):   # the single-row portions in the tile kernel, then as decode rows
+        keep = md["tile_seq"] >= nd
+        got = mx.sigmoid_attention(q.cuda(), kc.cuda(), vc.cuda(), g["block_tables"],
+                                   g["seq_kvlen"], g["seq_qstart"],
+                                   md["tile_seq"][keep].cuda(), md["tile_qoff"][keep].cuda(),
+                                   scale, cap, bias.cuda(), talk.cuda(), nd,
+                                   int(md["seq_kvlen"][:max(nd, 1)].max())).cpu().float()
+        err = (got - want).abs() / (want.abs() + want.pow(2).mean().sqrt())
+        bf = dt == torch.bfloat16
+        assert float(err.max()) < (4e-2 if bf else 2e-5), (nd, float(err.max()))
+        assert float(err.mean()) < (4e-3 if bf else 2e-6), (nd, float(err.mean()))
+
+
+@pytest.mark.parametrize("dt", DTYPES)
+@pytest.mark.parametrize("W", [40, 100, 1024, 4096, 33000])
+def test_post_norm(dt, W):
+    torch.manual_seed(2)
+    T = 9
+    x = 3 * torch.randn(T, W)
+    a, b = torch.randn(T, W).to(dt), torch.randn(T, W).to(dt)
+    w = (1 + 0.1 * torch.randn(W)).to(dt)
+    for bb in (b, None):
+        xr, xg = x.clone(), x.clone().cuda()
+        want = mref.post_norm(xr, 1.7, a, 0.6, bb, 0.9, w, 1e-5, dt)
+        got = mx.post_norm(xg, 1.7, a.cuda(), 0.6, None if bb is None else bb.cuda(), 0.9,
+                           w.cuda(), 1e-5, dt)
+        assert torch.allclose(xg.cpu(), xr, atol=2e-5, rtol=2e-5)
+        assert got.dtype == dt
+        assert torch.allclose(got.cpu().float(), want.float(), **tol(dt))
+
+
+@pytest.mark.parametrize("dt", DTYPES)
+@pytest.mark.parametrize("G,vdim,bs", [(2, 48, 16), (3, 20, 16), (1, 130, 8), (2, 9, 12)])
+def test_values_normed_mixed_and_temperature(dt, G, vdim, bs):
+    torch.manual_seed(3)
+    H, dim = 2 * G, 24
+    md = ragged(LENS, STARTS, SLOTS, bs=bs, width=20)
+    md["slot_mapping"][1] = -1
+    g = cuda(md)
+    T = int(md["seq_qstart"][-1])
+    P = torch.randn(T, H * dim + G * dim + G * vdim + 8).to(dt)
+    qn, kn = torch.randn(H * dim).to(dt), torch.randn(G * dim).to(dt)
+    first = torch.randn(T, G * vdim).to(dt)
+    table = mref.rotary_table(md["positions"], mx.inv_freq(10, 50.0, "cpu"), 1.3)
+    tg = mx.rotary_table(g["positions"], mx.inv_freq(10, 50.0, "cuda"), 1.3)
+    assert torch.allclose(tg.cpu(), table, atol=1e-5, rtol=1e-5)
+    cut = lambda t: (t[:, :H * dim], t[:, H * dim:(H + G) * dim],  # noqa: E731
+                     t[:, (H + G) * dim:(H + G) * dim + G * vdim])
+    for norm, fst in ((True, None), (True, first), (False, first), (False, None)):
+        kc, vc = ragged_pages(md, G, dim, vdim, bs, dt, 5)
+        kg, vg = kc.clone().cuda(), vc.clone().cuda()
+        vo, vog = torch.zeros(T, G * vdim, dtype=dt), torch.zeros(T, G * vdim, dtype=dt).cuda()
+        kw = dict(rotate_half_pairs=True, whole_norm=True, q_temp=(0.4, 7.0), v_norm=norm,
+                  v_lambda=0.3)
+        want = mref.qk_norm_rope_cache(*cut(P), qn, kn, 1e-5, md["positions"], md["slot_mapping"],
+                                       table, kc, vc, H, G, dim, vdim, v_first=fst, v_out=vo, **kw)
+        got = mx.qk_norm_rope_cache(*cut(P.cuda()), qn.cuda(), kn.cuda(), 1e-5, g["positions"],
+                                    g["slot_mapping"], tg, kg, vg, H, G, dim, vdim,
+                                    v_first=None if fst is None else fst.cuda(), v_out=vog, **kw)
+        assert torch.allclose(got.cpu().float(), want.float(), **tol(dt))
+        assert torch.allclose(kg.cpu().float(), kc.float(), **tol(dt))
+        assert torch.allclose(vg.cpu().float(), vc.float(), **tol(dt))
+        live = md["slot_mapping"][:T] >= 0
+        assert torch.allclose(vog.cpu().float()[live], vo.float()[live], **tol(dt))
+
+
+@pytest.mark.parametrize("dt", DTYPES)
+def test_gates_and_interleaved_latent_front_end(dt):
+    torch.manual_seed(4)
+    md = ragged(LENS, STARTS, SLOTS)
+    g = cuda(md)
+    T, H = int(md["seq_qstart"][-1]), 3
+    for dv in (16, 20):
+        o, wide = torch.randn(H, T, dv).to(dt), torch.randn(T, H * dv + 8).to(dt)
+        for gate in (wide[:, :H], wide[:, :H * dv]):
+            got = mx.head_gate(o.cuda(), wide.cuda()[:, :gate.shape[1]])
+            assert torch.allclose(got.cpu().float(), mref.head_gate(o, gate).float(), **tol(dt))
+    # interleaved pairs on the rotated part of row-strided queries
+    rank, rot, qd, bs = 24, 12, 16, 16
+    wide = torch.randn(T, H * (qd + rot) + 8).to(dt)
+    q_lat, kvx = torch.randn(H, T, rank).to(dt), torch.randn(T, rank + rot).to(dt)
+    cn = torch.randn(rank).to(dt)
+    table = mref.rotary_table(md["positions"], mx.inv_freq(10, 50.0, "cpu"))
+    res = []
+    for dev, m_ in (("cpu", md), ("cuda", g)):
+        qx = wide.to(dev)[:, :H * (qd + rot)].unflatten(1, (H, qd + rot))
+        kc = torch.zeros(md["num_pages"], 1, bs, rank + rot, dtype=dt, device=dev)
+        vc = torch.zeros(md["num_pages"], 1, rank, bs, dtype=dt, device=dev)
+        q = mx.latent_rope_cache(q_lat.to(dev), qx, kvx.to(dev), cn.to(dev), 1e-5,
+                                 m_["slot_mapping"], table.to(dev), kc, vc, False)
+        res.append([t.cpu().float() for t in (q, kc, vc)])
+    for a, b in zip(*res):
+        assert torch.allclose(a, b, **tol(dt))
+    # per-head gate in the attention kernels' store: tiles and decode rows
+    for dim, vdim in ((32, 64), (20, 12)):
+        G = 3
+        q = torch.randn(T, H, dim).to(dt)
+        kc, vc = ragged_pages(md, G, dim, vdim, 16, dt)
+        gate = torch.randn(T, 11).to(dt)
+        want = mref.sink_attention(q, kc, vc, md["block_tables"], md["seq_kvlen"],
+                                   md["seq_qstart"], 0.2, False, None, 9, gate[:, 8:])
+        keep = md["tile_seq"] >= 2
+        got = mx.sink_attention(q.cuda(), kc.cuda(), vc.cuda(), g["block_tables"], g["seq_kvlen"],
+                                g["seq_qstart"], md["tile_seq"][keep].cuda(),
+                                md["tile_qoff"][keep].cuda(), 0.2, False, 2, 71, None, 9,
+                                gate.cuda()[:, 8:])
+        assert torch.allclose(got.cpu().float(), want.float(), **tol(dt))
+
+
+@pytest.mark.parametrize("E,top", [(16, 2), (5, 5), (70, 3), (300, 4), (3, 1)])
+def test_route_by_logit(E, top):
+    logits = 40 * torch.randn(50, E)
+    logits[3] -= 500.0          # a softmax over the row would leave no second choice
+    logits[3, 1] += 900.0
+    got = mx.moe_route(logits.cuda(), top, "logit")
+    want = mref.moe_route(logits, top, "logit")
+    assert torch.equal(got[0].cpu(), want[0])
+    assert torch.allclose(got[1].cpu(), want[1], atol=1e-6, rtol=1e-5)
