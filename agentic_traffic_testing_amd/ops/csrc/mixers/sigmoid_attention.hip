@@ -20,8 +20,9 @@
 //        [slot][token][key];
 //     C  O^T[16 channels x 16 tokens] += V^T . mixed^T (V^T rows straight from the pages).
 //   B needs A of all waves and C needs B of all waves; C of a tile and A of the next share one
-//   barrier interval, so a tile costs two barriers.  Row strides and an XOR of the 16-byte chunk
-//   with bits of the token keep the LDS accesses conflict-free.
+//   barrier interval, so a tile costs two barriers (which order LDS only: the V fragments of the
+//   tile are in flight during B, the first K fragments of the next one during C).  The LDS
+//   images are XOR-swizzled (sg_place) so that no access of any phase has a bank conflict.
 // * matrix-core decode kernel (bf16, dim % 8 == 0, dim <= 256, vdim % 16 == 0, H <= 64): one
 //   workgroup per (sequence, 64-key partition), columns = the query heads of a KV head; the mix
 //   runs on the VALU in fp32; the partition's sums go to `part`, a combine kernel adds them.
@@ -42,8 +43,11 @@ constexpr int kSgTok = 16;      // query tokens per workgroup (matrix-core prefi
 constexpr int kSgKeys = 32;     // keys per tile
 constexpr int kSgPart = 64;     // keys per decode partition
 constexpr int kSgSlots = 32;    // head slots
-constexpr int kSgRow = kSgTok * 32 + 8;   // LDS row of 16 tokens x 32 bf16, padded by 16 bytes
+constexpr int kSgRow = kSgTok * 32;       // LDS row (of a key, of a slot): 16 tokens x 32 bf16
 constexpr int kSgAcc = 64;      // accumulators per thread of the rows kernel
+// heads per wave whose Q fragments live in LDS: the widest form is short of registers (it uses
+// all of a CU's 160 KB)
+__host__ __device__ constexpr int sg_q_lds(int HW, int ND) { return HW == 4 && ND == 4 ? 2 : 0; }
 constexpr float kLog2e = 1.44269504088896341f;
 
 struct SigArgs {
@@ -82,23 +86,45 @@ __device__ __forceinline__ sg_bf16x8 zero_frag() {
   const sg_u32x4 z = {0u, 0u, 0u, 0u};
   return __builtin_bit_cast(sg_bf16x8, z);
 }
-// 8 keys of a V^T row starting at key t8; keys at or past kend become zero
-__device__ __forceinline__ sg_bf16x8 ld_v(const __bf16* p, int t8, int kend) {
-  if (t8 >= kend) return zero_frag();
-  sg_bf16x8 v = ld_frag(p);
-  if (t8 + 8 > kend) {
-#pragma unroll
-    for (int j = 0; j < 8; ++j)
-      if (t8 + j >= kend) v[j] = static_cast<__bf16>(0.f);
-  }
+// Place of (row, token, 16-byte chunk) in an LDS image of rows of 16 tokens x 4 chunks.  The token is
+// XORed with the row and the chunk with the token's place, so that neither 16 tokens of a row nor
+// 16 rows of a token share a bank.
+__device__ __forceinline__ int sg_place(int row, int t, int chunk) {
+  const int p = t ^ (row & 15);
+  return row * kSgRow + p * 32 + ((chunk ^ (p >> 2)) << 3);
+}
+
+// A copy the compiler knows nothing about: what is computed from it stays inside the loop instead of
+// being hoisted into registers that the accumulators need.
+__device__ __forceinline__ int fresh(int v) {
+  asm volatile("" : "+v"(v));
   return v;
 }
 
-template <int HW, int ND, int NV, bool CAP>   // dim <= 32 ND, vdim <= 16 NV, H <= 8 HW
+// Keys at or past kend of the 8 that start at t8 become zero (stale cache contents).
+__device__ __forceinline__ sg_bf16x8 keep_keys(sg_bf16x8 v, int t8, int kend) {
+#pragma unroll
+  for (int j = 0; j < 8; ++j)
+    if (t8 + j >= kend) v[j] = static_cast<__bf16>(0.f);
+  return v;
+}
+// Workgroup barrier that orders LDS only: global loads in flight stay in flight.
+__device__ __forceinline__ void lds_barrier() {
+  __builtin_amdgcn_sched_barrier(0);
+  asm volatile("s_waitcnt lgkmcnt(0)\n\ts_barrier" ::: "memory");
+  __builtin_amdgcn_sched_barrier(0);
+}
+
+// ONE: the heads of a wave share one KV head (H / G is a multiple of HW), so its K and V fragments
+// are loaded once per tile, ahead of their use.
+template <int HW, int ND, int NV, bool CAP, bool ONE>   // dim <= 32 ND, vdim <= 16 NV, H <= 8 HW
 __global__ void __launch_bounds__(512)
 sigmoid_attention_mfma_kernel(__bf16* __restrict__ out, const __bf16* __restrict__ q,
                               const __bf16* __restrict__ k_cache,
                               const __bf16* __restrict__ v_cache, SigArgs a) {
+  constexpr int QL = sg_q_lds(HW, ND), QR = HW - QL;     // heads with Q in LDS / in registers
+  constexpr int QS = 32 * ND;                            // LDS row of one token's Q
+  constexpr int NF = HW * NV >= 32 ? NV / 2 : NV;        // V fragments in flight (registers)
   extern __shared__ __attribute__((aligned(16))) char sg_smem[];
   __bf16* w_hi = reinterpret_cast<__bf16*>(sg_smem);     // [32 keys][kSgRow]
   __bf16* w_lo = w_hi + kSgKeys * kSgRow;
@@ -119,19 +145,29 @@ sigmoid_attention_mfma_kernel(__bf16* __restrict__ out, const __bf16* __restrict
   const int h0 = w * HW;
   const bool wave_on = h0 < H;
   const int qpos = pos0 + r;
-  const int tswz = (r >> 2) & 3;
+  // head QR + e of the wave in LDS: this lane's row of the e-th 16-token block, chunks XORed with r
+  __bf16* q_rows = mixed + kSgSlots * kSgRow + (w * QL * kSgTok + r) * QS;
+  auto q_lds = [&](int e, int st, int rr) {
+    return q_rows + e * kSgTok * QS + (((st * 4 + c) ^ (rr & (4 * ND - 1))) << 3);
+  };
 
-  sg_bf16x8 qf[HW][ND];
+  // Q fragments; channels past dim, tokens past ntok and heads past H are zero
+  sg_bf16x8 qf[QR > 0 ? QR : 1][ND];
   float k3[HW];
 #pragma unroll
   for (int hh = 0; hh < HW; ++hh) {
     const int h = h0 + hh;
-    k3[hh] = h < H ? -((CAP ? a.cap : 0.f) + a.bias[h]) * kLog2e : 0.f;
+    // a head past H: exp2(inf) makes every weight an exact zero
+    k3[hh] = h < H ? -((CAP ? a.cap : 0.f) + a.bias[h]) * kLog2e : INFINITY;
 #pragma unroll
     for (int st = 0; st < ND; ++st) {
-      qf[hh][st] = zero_frag();
+      sg_bf16x8 f = zero_frag();
       if (r < ntok && h < H && st * 32 + 8 * c < dim)
-        qf[hh][st] = ld_frag(q + (static_cast<int64_t>(row0 + qo + r) * H + h) * dim + st * 32 + 8 * c);
+        f = ld_frag(q + (static_cast<int64_t>(row0 + qo + r) * H + h) * dim + st * 32 + 8 * c);
+      if (hh < QR)
+        qf[hh < QR ? hh : 0][st] = f;
+      else
+        *reinterpret_cast<sg_bf16x8*>(q_lds(hh - QR, st, r)) = f;   // read back by this lane only
     }
   }
   const float k1 = CAP ? 2.0f * kLog2e * a.scale / a.cap : -kLog2e * a.scale;
@@ -157,91 +193,125 @@ sigmoid_attention_mfma_kernel(__bf16* __restrict__ out, const __bf16* __restrict
 #pragma unroll
     for (int vt = 0; vt < NV; ++vt) O[hh][vt] = sg_f32x4{0.f, 0.f, 0.f, 0.f};
 
+  // Addresses are clamped instead of predicated: a key past the end reads the last key (its
+  // weight is masked), a channel group past dim reads group 0 (its Q is zero), a channel tile
+  // past vdim reads the last one (never stored), a head past H the last one (zero weights).
   const int* bt = a.block_tables + static_cast<int64_t>(s) * a.bt_width;
   const int64_t kpage = static_cast<int64_t>(G) * bs * dim, vpage = static_cast<int64_t>(G) * vdim * bs;
-  const int shift = a.bs_shift, bmask = bs - 1;
-  auto page_at = [&](int key) -> int64_t { return key < kend ? bt[key >> shift] : 0; };
-
-  auto scores = [&](int k0, int64_t pg0, int64_t pg1) {
-    if (!wave_on) {
-      if (k0 == 0) {   // this wave's slots never hold a head: zero them once
-        const sg_bf16x4 z = {static_cast<__bf16>(0.f), static_cast<__bf16>(0.f),
-                             static_cast<__bf16>(0.f), static_cast<__bf16>(0.f)};
-        for (int i = 0; i < 8; ++i) {
-          const int key = (i >> 2) * 16 + 4 * c + (i & 3);
-          const int o = key * kSgRow + r * 32 + (((w >> 1) ^ tswz) << 3) + (w & 1) * 4;
-          *reinterpret_cast<sg_bf16x4*>(w_hi + o) = z;
-          *reinterpret_cast<sg_bf16x4*>(w_lo + o) = z;
-        }
-      }
-      return;
-    }
-    const bool edge = k0 + kSgKeys - 1 > pos0;   // some key lies after the first query token
+  const int shift = a.bs_shift, bmask = bs - 1, last = kend - 1;
+  auto kv_head = [&](int hh) { return min(h0 + hh, H - 1) / rep; };
+  auto page_at = [&](int key) { return bt[min(key, last) >> shift]; };
+  const int g0 = kv_head(0);
+  int koff[ND];
 #pragma unroll
-    for (int sub = 0; sub < 2; ++sub) {
-      const int key = k0 + sub * 16 + r;
-      const __bf16* kb = k_cache + (sub ? pg1 : pg0) * kpage + static_cast<int64_t>(key & bmask) * dim + 8 * c;
-      sg_bf16x8 kf[ND];
-      float wt[4][4];
+  for (int st = 0; st < ND; ++st) koff[st] = st * 32 + 8 * c < dim ? st * 32 + 8 * c : 0;
+
+  auto load_k = [&](sg_bf16x8 (&kf)[ND], int page, int key, int g) {
+    const __bf16* kb = k_cache + page * kpage +
+                       static_cast<int64_t>(g * bs + (min(key, last) & bmask)) * dim;
+#pragma unroll
+    for (int st = 0; st < ND; ++st) kf[st] = ld_frag(kb + koff[st]);
+  };
+  auto head_scores = [&](const sg_bf16x8 (&kf)[ND], int hh, int rr) {
+    sg_f32x4 S = {0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+    for (int st = 0; st < ND; ++st) {
+      const sg_bf16x8 f = hh < QR ? qf[hh < QR ? hh : 0][st] : ld_frag(q_lds(hh - QR, st, rr));
+      S = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kf[st], f, S, 0, 0, 0);
+    }
+    return S;
+  };
+  // weights of keys k0 + 16 sub .. + 15 for the wave's heads, into the LDS image
+  auto weights = [&](int k0, int sub, const sg_f32x4 (&S)[HW]) {
+    const int kb = k0 + sub * 16 + 4 * c;
+    const bool edge = k0 + kSgKeys - 1 > pos0;   // some key lies after the first query token
+    const int rr = fresh(r);
+#pragma unroll
+    for (int i = 0; i < 4; ++i) {
+      sg_bf16x4 hi, lo;
 #pragma unroll
       for (int hh = 0; hh < 4; ++hh) {
-        if (hh >= HW) {
-#pragma unroll
-          for (int i = 0; i < 4; ++i) wt[hh][i] = 0.f;
-          continue;
+        float x = 0.f;
+        if (hh < HW) {
+          x = sig_weight<CAP>(S[hh < HW ? hh : 0][i], k1, k2, k3[hh < HW ? hh : 0]);
+          if (edge && kb + i > qpos) x = 0.f;
         }
-        const int h = h0 + hh;
-        const int g = h / rep;
-        if (h < H && (hh == 0 || g != (h - 1) / rep)) {   // wave-uniform: a new KV head
-#pragma unroll
-          for (int st = 0; st < ND; ++st) {
-            kf[st] = zero_frag();
-            if (key < kend && st * 32 + 8 * c < dim)
-              kf[st] = ld_frag(kb + static_cast<int64_t>(g) * bs * dim + st * 32);
-          }
-        }
-        sg_f32x4 S = {0.f, 0.f, 0.f, 0.f};
-#pragma unroll
-        for (int st = 0; st < ND; ++st)
-          S = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kf[st], qf[hh < HW ? hh : 0][st], S, 0, 0, 0);
-        const float b = k3[hh < HW ? hh : 0];
-#pragma unroll
-        for (int i = 0; i < 4; ++i) {
-          float x = h < H ? sig_weight<CAP>(S[i], k1, k2, b) : 0.f;
-          if (edge && k0 + sub * 16 + 4 * c + i > qpos) x = 0.f;
-          wt[hh][i] = x;
-        }
+        hi[hh] = static_cast<__bf16>(x);
+        lo[hh] = static_cast<__bf16>(x - static_cast<float>(hi[hh]));
       }
+      const int o = sg_place(sub * 16 + 4 * c + i, rr, w >> 1) + (w & 1) * 4;
+      *reinterpret_cast<sg_bf16x4*>(w_hi + o) = hi;
+      *reinterpret_cast<sg_bf16x4*>(w_lo + o) = lo;
+    }
+  };
+
+  sg_bf16x8 ka[ND];   // ONE: K of the next tile's first 16 keys, in flight
+  auto scores = [&](int k0, int pg0, int pg1) {
+    const int rr = fresh(r);
+    if (ONE) {
+      sg_bf16x8 kb[ND];
+      sg_f32x4 S[HW];
 #pragma unroll
-      for (int i = 0; i < 4; ++i) {
-        const int kk = sub * 16 + 4 * c + i;
-        const int o = kk * kSgRow + r * 32 + (((w >> 1) ^ tswz) << 3) + (w & 1) * 4;
-        sg_bf16x4 hi, lo;
+      for (int hh = 0; hh < HW; ++hh) S[hh] = head_scores(ka, hh, rr);
+      // the second half's K loads take over the first half's registers and land during its weights
+      __builtin_amdgcn_sched_barrier(0);
+      load_k(kb, pg1, k0 + 16 + r, g0);
+      __builtin_amdgcn_sched_barrier(0);
+      weights(k0, 0, S);
+      __builtin_amdgcn_sched_barrier(0);
 #pragma unroll
-        for (int hh = 0; hh < 4; ++hh) {
-          hi[hh] = static_cast<__bf16>(wt[hh][i]);
-          lo[hh] = static_cast<__bf16>(wt[hh][i] - static_cast<float>(hi[hh]));
+      for (int hh = 0; hh < HW; ++hh) S[hh] = head_scores(kb, hh, rr);
+      weights(k0, 1, S);
+    } else {
+#pragma unroll
+      for (int sub = 0; sub < 2; ++sub) {
+        sg_f32x4 S[HW];
+#pragma unroll
+        for (int hh = 0; hh < HW; ++hh) {
+          sg_bf16x8 kf[ND];
+          load_k(kf, sub ? pg1 : pg0, k0 + sub * 16 + r, kv_head(hh));
+          S[hh] = head_scores(kf, hh, rr);
         }
-        *reinterpret_cast<sg_bf16x4*>(w_hi + o) = hi;
-        *reinterpret_cast<sg_bf16x4*>(w_lo + o) = lo;
+        weights(k0, sub, S);
       }
     }
   };
 
-  int64_t pk0 = page_at(r), pk1 = page_at(16 + r), pv = page_at(8 * c);
-  scores(0, pk0, pk1);
+  int pk0 = page_at(r), pk1 = page_at(16 + r), pv = page_at(8 * c);
+  if (wave_on) {
+    if (ONE) load_k(ka, pk0, r, g0);
+    scores(0, pk0, pk1);
+  } else {   // this wave's slots never hold a head: zero them once
+    const sg_bf16x4 z = {static_cast<__bf16>(0.f), static_cast<__bf16>(0.f),
+                         static_cast<__bf16>(0.f), static_cast<__bf16>(0.f)};
+    for (int key = c; key < kSgKeys; key += 4) {
+      const int o = sg_place(key, r, w >> 1) + (w & 1) * 4;
+      *reinterpret_cast<sg_bf16x4*>(w_hi + o) = z;
+      *reinterpret_cast<sg_bf16x4*>(w_lo + o) = z;
+    }
+  }
+  pk0 = page_at(kSgKeys + r);
+  pk1 = page_at(kSgKeys + 16 + r);
   for (int k0 = 0; k0 < kend; k0 += kSgKeys) {
-    __syncthreads();
-    const int nk = k0 + kSgKeys;
-    pk0 = page_at(nk + r);
-    pk1 = page_at(nk + 16 + r);
+    const int nk = k0 + kSgKeys, t8 = k0 + 8 * c;
+    const __bf16* vb = v_cache + pv * vpage + (min(t8, last) & bmask & ~7) + static_cast<int64_t>(r) * bs;
+    sg_bf16x8 vf[NF];
+    auto load_v = [&](int vt0) {
+#pragma unroll
+      for (int e = 0; e < NF; ++e)
+        vf[e] = ld_frag(vb + static_cast<int64_t>(g0 * vdim + min(vt0 + e, nv - 1) * 16) * bs);
+    };
+    if (ONE && wave_on) load_v(0);
+    pv = page_at(nk + 8 * c);
+    lds_barrier();
+    const int rb = fresh(r);
     // B: the wave mixes the pairs of tokens 2 w and 2 w + 1
 #pragma unroll
     for (int tt = 0; tt < 2; ++tt) {
-      const int t = 2 * w + tt, swz = (t >> 2) & 3;
+      const int t = 2 * w + tt;
 #pragma unroll
       for (int half = 0; half < 2; ++half) {
-        const int o = (half * 16 + r) * kSgRow + t * 32 + ((c ^ swz) << 3);
+        const int o = sg_place(half * 16 + rb, t, c);
         const sg_bf16x8 ah = ld_frag(w_hi + o), al = ld_frag(w_lo + o);
 #pragma unroll
         for (int ht = 0; ht < 2; ++ht) {
@@ -252,39 +322,57 @@ sigmoid_attention_mfma_kernel(__bf16* __restrict__ out, const __bf16* __restrict
             sg_bf16x4 e;
 #pragma unroll
             for (int i = 0; i < 4; ++i) e[i] = static_cast<__bf16>(D[i]);
-            *reinterpret_cast<sg_bf16x4*>(mixed + (ht * 16 + r) * kSgRow + t * 32 +
-                                          (((half * 2 + (c >> 1)) ^ swz) << 3) + (c & 1) * 4) = e;
+            *reinterpret_cast<sg_bf16x4*>(mixed + sg_place(ht * 16 + rb, t, half * 2 + (c >> 1)) +
+                                          (c & 1) * 4) = e;
           }
         }
       }
     }
-    __syncthreads();
+    lds_barrier();
     if (wave_on) {   // C
-      const int t8 = k0 + 8 * c;
-      sg_bf16x8 pf[HW];
+      const bool tail = nk > kend;
+      const int rc = fresh(r);
+      if (ONE) {
 #pragma unroll
-      for (int hh = 0; hh < HW; ++hh)
-        pf[hh] = ld_frag(mixed + (4 * w + hh) * kSgRow + r * 32 + ((c ^ tswz) << 3));
-      const __bf16* vb = v_cache + pv * vpage + (t8 & bmask) + static_cast<int64_t>(r) * bs;
+        for (int vt0 = 0; vt0 < NV; vt0 += NF) {
+          if (vt0 > 0) load_v(vt0);
+          if (vt0 + NF >= NV && NF < NV) load_k(ka, pk0, nk + r, g0);
+          if (tail) {
 #pragma unroll
-      for (int vt = 0; vt < NV; ++vt) {
-        if (vt < nv) {
-          sg_bf16x8 vf = zero_frag();
+            for (int e = 0; e < NF; ++e) vf[e] = keep_keys(vf[e], t8, kend);
+          }
 #pragma unroll
           for (int hh = 0; hh < HW; ++hh) {
-            const int h = h0 + hh;
-            if (h < H) {
-              const int g = h / rep;
-              if (hh == 0 || g != (h - 1) / rep)
-                vf = ld_v(vb + (static_cast<int64_t>(g) * vdim + vt * 16) * bs, t8, kend);
-              O[hh][vt] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(vf, pf[hh], O[hh][vt], 0, 0, 0);
-            }
+            const sg_bf16x8 pf = ld_frag(mixed + sg_place(4 * w + hh, rc, c));
+#pragma unroll
+            for (int e = 0; e < NF; ++e)
+              O[hh][vt0 + e] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(vf[e], pf, O[hh][vt0 + e], 0, 0, 0);
           }
+          __builtin_amdgcn_sched_barrier(0);
+        }
+        if (NF == NV) load_k(ka, pk0, nk + r, g0);
+        __builtin_amdgcn_sched_barrier(0);
+      } else {
+#pragma unroll
+        for (int hh = 0; hh < HW; ++hh) {
+          const sg_bf16x8 pf = ld_frag(mixed + sg_place(4 * w + hh, rc, c));
+          const __bf16* vh = vb + static_cast<int64_t>(kv_head(hh)) * vdim * bs;
+          sg_bf16x8 vg[NV];
+#pragma unroll
+          for (int vt = 0; vt < NV; ++vt) vg[vt] = ld_frag(vh + static_cast<int64_t>(min(vt, nv - 1)) * 16 * bs);
+          if (tail) {
+#pragma unroll
+            for (int vt = 0; vt < NV; ++vt) vg[vt] = keep_keys(vg[vt], t8, kend);
+          }
+#pragma unroll
+          for (int vt = 0; vt < NV; ++vt)
+            O[hh][vt] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(vg[vt], pf, O[hh][vt], 0, 0, 0);
         }
       }
+      if (nk < kend) scores(nk, pk0, pk1);
     }
-    pv = page_at(nk + 8 * c);
-    if (nk < kend) scores(nk, pk0, pk1);
+    pk0 = page_at(nk + kSgKeys + r);
+    pk1 = page_at(nk + kSgKeys + 16 + r);
   }
   if (!wave_on || r >= ntok) return;
 #pragma unroll
@@ -305,21 +393,28 @@ sigmoid_attention_mfma_kernel(__bf16* __restrict__ out, const __bf16* __restrict
   }
 }
 
-// One workgroup of four waves per (decode sequence, 64-key partition), all heads.
+// One workgroup of eight waves per (decode sequence, 64-key partition), all heads.
+constexpr int kSgMixRow = kSgPart + 8;
+// dynamic LDS: mixed weights bf16 [H][72], weights fp32 [64 keys][H + 1], talk fp32 [H][H]
+__host__ __device__ constexpr size_t sg_decode_smem(int H) {
+  return sizeof(__bf16) * H * kSgMixRow + sizeof(float) * (kSgPart * (H + 1) + H * H);
+}
+
 template <int ND, bool CAP>   // dim <= 32 ND
-__global__ void __launch_bounds__(256)
+__global__ void __launch_bounds__(512)
 sigmoid_attention_decode_kernel(const __bf16* __restrict__ q, const __bf16* __restrict__ k_cache,
                                 const __bf16* __restrict__ v_cache, SigArgs a) {
   extern __shared__ __attribute__((aligned(16))) char sg_smem[];
   const int H = a.H, G = a.G, dim = a.dim, vdim = a.vdim, bs = a.block_size, HS = H + 1;
-  constexpr int PR = kSgPart + 8;
-  __bf16* mixed = reinterpret_cast<__bf16*>(sg_smem);                       // [H][72]
-  float* wts = reinterpret_cast<float*>(sg_smem + sizeof(__bf16) * H * PR); // [64 keys][H + 1]
+  constexpr int PR = kSgMixRow;
+  __bf16* mixed = reinterpret_cast<__bf16*>(sg_smem);
+  float* wts = reinterpret_cast<float*>(sg_smem + sizeof(__bf16) * H * PR);
+  float* talk = wts + kSgPart * HS;
   const int s = blockIdx.x, kbeg = blockIdx.y * kSgPart;
   const int kvlen = a.seq_kvlen[s];
   const int kend = min(kvlen, kbeg + kSgPart);
   if (kbeg >= kend) return;
-  const int rep = H / G, ct = (rep + 15) >> 4;
+  const int rep = H / G, ct = (rep + 15) >> 4, last = kend - 1;
   const int lane = threadIdx.x & 63, r = lane & 15, c = lane >> 4;
   const int w = __builtin_amdgcn_readfirstlane(static_cast<int>(threadIdx.x) >> 6);
   const int* bt = a.block_tables + static_cast<int64_t>(s) * a.bt_width;
@@ -327,30 +422,41 @@ sigmoid_attention_decode_kernel(const __bf16* __restrict__ q, const __bf16* __re
   const float k1 = CAP ? 2.0f * kLog2e * a.scale / a.cap : -kLog2e * a.scale;
   const float k2 = 2.0f * a.cap * kLog2e;
   const int shift = a.bs_shift, bmask = bs - 1;
-  // wave w scores keys 16 w .. 16 w + 15 of the partition for every KV head
+  // the V pages of this lane's key groups (clamped like every address here)
+  const __bf16* vb[2];
+#pragma unroll
+  for (int ks = 0; ks < 2; ++ks) {
+    const int t8 = min(kbeg + ks * 32 + 8 * c, last);
+    vb[ks] = v_cache + static_cast<int64_t>(bt[t8 >> shift]) * G * vdim * bs + (t8 & bmask & ~7) +
+             static_cast<int64_t>(r) * bs;
+  }
+  for (int i = threadIdx.x; i < H * H; i += 512) talk[i] = a.talk[i];
+  // waves w and w + 4 score keys 16 (w & 3) .. + 15 of the partition, every other KV head each
   {
-    const int key = kbeg + 16 * w + r;
-    const bool live = key < kend;
-    const __bf16* kb = k_cache + (live ? static_cast<int64_t>(bt[key >> shift]) : 0) * G * bs * dim +
-                       static_cast<int64_t>(key & bmask) * dim + 8 * c;
-    for (int j = 0; j < G * ct; ++j) {
+    const int key = min(kbeg + 16 * (w & 3) + r, last);
+    const __bf16* kb = k_cache + static_cast<int64_t>(bt[key >> shift]) * G * bs * dim +
+                       static_cast<int64_t>(key & bmask) * dim;
+#pragma unroll 2
+    for (int j = w >> 2; j < G * ct; j += 2) {
       const int g = j / ct, hl = (j - g * ct) * 16 + r, h = g * rep + hl;
       const bool hok = hl < rep;
-      sg_f32x4 S = {0.f, 0.f, 0.f, 0.f};
+      const __bf16* qr = q + (row * H + min(h, H - 1)) * dim;
+      sg_bf16x8 kf[ND], qf[ND];
 #pragma unroll
       for (int st = 0; st < ND; ++st) {
-        sg_bf16x8 kf = zero_frag(), qf = zero_frag();
-        if (st * 32 + 8 * c < dim) {
-          if (live) kf = ld_frag(kb + static_cast<int64_t>(g) * bs * dim + st * 32);
-          if (hok) qf = ld_frag(q + (row * H + h) * dim + st * 32 + 8 * c);
-        }
-        S = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kf, qf, S, 0, 0, 0);
+        const int ch = st * 32 + 8 * c;
+        kf[st] = ld_frag(kb + static_cast<int64_t>(g) * bs * dim + (ch < dim ? ch : 0));
+        qf[st] = ch < dim ? ld_frag(qr + ch) : zero_frag();
       }
+      const float k3 = -((CAP ? a.cap : 0.f) + a.bias[min(h, H - 1)]) * kLog2e;
+      sg_f32x4 S = {0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+      for (int st = 0; st < ND; ++st)
+        S = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kf[st], qf[st], S, 0, 0, 0);
       if (hok) {
-        const float k3 = -((CAP ? a.cap : 0.f) + a.bias[h]) * kLog2e;
 #pragma unroll
         for (int i = 0; i < 4; ++i) {
-          const int kk = 16 * w + 4 * c + i;
+          const int kk = 16 * (w & 3) + 4 * c + i;
           wts[kk * HS + h] = kbeg + kk < kend ? sig_weight<CAP>(S[i], k1, k2, k3) : 0.f;
         }
       }
@@ -358,11 +464,12 @@ sigmoid_attention_decode_kernel(const __bf16* __restrict__ q, const __bf16* __re
   }
   __syncthreads();
   // lane = key, four output heads per pass of a wave
-  for (int hb = 4 * w; hb < H; hb += 16) {
+  for (int hb = 4 * w; hb < H; hb += 32) {
     float m[4] = {0.f, 0.f, 0.f, 0.f};
     const float* tr[4];
 #pragma unroll
-    for (int e = 0; e < 4; ++e) tr[e] = a.talk + static_cast<int64_t>(min(hb + e, H - 1)) * H;
+    for (int e = 0; e < 4; ++e) tr[e] = talk + min(hb + e, H - 1) * H;
+#pragma unroll 4
     for (int g = 0; g < H; ++g) {
       const float x = wts[lane * HS + g];
 #pragma unroll
@@ -374,21 +481,22 @@ sigmoid_attention_decode_kernel(const __bf16* __restrict__ q, const __bf16* __re
   }
   __syncthreads();
   const int nv = vdim >> 4;
-  for (int j = w; j < G * ct * nv; j += 4) {
+#pragma unroll 4
+  for (int j = w; j < G * ct * nv; j += 8) {
     const int vt = j % nv, gc = j / nv;
     const int g = gc / ct, hl = (gc - g * ct) * 16 + r, h = g * rep + hl;
-    sg_f32x4 O = {0.f, 0.f, 0.f, 0.f};
+    const int64_t vo = static_cast<int64_t>(g * vdim + vt * 16) * bs;
+    sg_bf16x8 vf[2], pf[2];
 #pragma unroll
     for (int ks = 0; ks < 2; ++ks) {
-      const int t8 = kbeg + ks * 32 + 8 * c;
-      sg_bf16x8 vf = zero_frag();
-      if (t8 < kend)
-        vf = ld_v(v_cache + (static_cast<int64_t>(bt[t8 >> shift]) * G + g) * vdim * bs +
-                      static_cast<int64_t>(vt * 16 + r) * bs + (t8 & bmask),
-                  t8, kend);
-      const sg_bf16x8 pf = hl < rep ? ld_frag(mixed + h * PR + ks * 32 + 8 * c) : zero_frag();
-      O = __builtin_amdgcn_mfma_f32_16x16x32_bf16(vf, pf, O, 0, 0, 0);
+      vf[ks] = ld_frag(vb[ks] + vo);
+      pf[ks] = hl < rep ? ld_frag(mixed + h * PR + ks * 32 + 8 * c) : zero_frag();
     }
+    sg_f32x4 O = {0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+    for (int ks = 0; ks < 2; ++ks)
+      O = __builtin_amdgcn_mfma_f32_16x16x32_bf16(keep_keys(vf[ks], kbeg + ks * 32 + 8 * c, kend),
+                                                  pf[ks], O, 0, 0, 0);
     if (hl < rep)
       *reinterpret_cast<sg_f32x4*>(a.part + ((static_cast<int64_t>(s) * H + h) * a.max_parts +
                                              blockIdx.y) * vdim + vt * 16 + 4 * c) = O;
@@ -521,27 +629,39 @@ int sg_smem_opt_in(K kernel, size_t smem) {
                                               static_cast<int>(smem)));
 }
 
-template <int HW, int ND, int NV, bool CAP>
+template <int HW, int ND, int NV, bool CAP, bool ONE>
 int sg_launch_prefill(void* out, const void* q, const void* k, const void* v, const SigArgs& a,
                       int num_tiles, hipStream_t st) {
-  const size_t smem = sizeof(__bf16) * (2 * kSgKeys + kSgSlots) * kSgRow;
+  const size_t smem = sizeof(__bf16) * ((2 * kSgKeys + kSgSlots) * kSgRow +
+                                        sg_q_lds(HW, ND) * 8 * kSgTok * 32 * ND);
+  static_assert(sizeof(__bf16) * (3 * 32 * 512 + 2 * 8 * 16 * 128) == 160 * 1024, "all of the LDS");
   static bool opted = false;
   if (!opted) {
-    if (int rc = sg_smem_opt_in(sigmoid_attention_mfma_kernel<HW, ND, NV, CAP>, smem)) return rc;
+    if (int rc = sg_smem_opt_in(sigmoid_attention_mfma_kernel<HW, ND, NV, CAP, ONE>, smem)) return rc;
     opted = true;
   }
-  hipLaunchKernelGGL((sigmoid_attention_mfma_kernel<HW, ND, NV, CAP>),
+  hipLaunchKernelGGL((sigmoid_attention_mfma_kernel<HW, ND, NV, CAP, ONE>),
                      dim3(num_tiles * (kSgTile / kSgTok)), dim3(512), smem, st,
                      static_cast<__bf16*>(out), static_cast<const __bf16*>(q),
                      static_cast<const __bf16*>(k), static_cast<const __bf16*>(v), a);
   return static_cast<int>(hipGetLastError());
 }
 
+template <int HW, int ND, int NV, bool CAP>
+int sg_prefill_kv(void* out, const void* q, const void* k, const void* v, const SigArgs& a,
+                  int num_tiles, hipStream_t st) {
+  if constexpr (HW > 1) {
+    if ((a.H / a.G) % HW != 0)
+      return sg_launch_prefill<HW, ND, NV, CAP, false>(out, q, k, v, a, num_tiles, st);
+  }
+  return sg_launch_prefill<HW, ND, NV, CAP, true>(out, q, k, v, a, num_tiles, st);
+}
+
 template <int HW, bool CAP>
 int sg_prefill_dims(void* out, const void* q, const void* k, const void* v, const SigArgs& a,
                     int num_tiles, hipStream_t st) {
-  if (a.dim <= 64 && a.vdim <= 64) return sg_launch_prefill<HW, 2, 4, CAP>(out, q, k, v, a, num_tiles, st);
-  return sg_launch_prefill<HW, 4, 8, CAP>(out, q, k, v, a, num_tiles, st);
+  if (a.dim <= 64 && a.vdim <= 64) return sg_prefill_kv<HW, 2, 4, CAP>(out, q, k, v, a, num_tiles, st);
+  return sg_prefill_kv<HW, 4, 8, CAP>(out, q, k, v, a, num_tiles, st);
 }
 
 template <bool CAP>
@@ -558,9 +678,9 @@ int sg_prefill(void* out, const void* q, const void* k, const void* v, const Sig
 template <int ND, bool CAP>
 void sg_launch_decode(const void* q, const void* k, const void* v, const SigArgs& a,
                       int num_decode, int parts, hipStream_t st) {
-  // H <= 64: at most 9 KB of mixed weights and 17 KB of weights
-  const size_t smem = sizeof(__bf16) * a.H * (kSgPart + 8) + sizeof(float) * kSgPart * (a.H + 1);
-  hipLaunchKernelGGL((sigmoid_attention_decode_kernel<ND, CAP>), dim3(num_decode, parts), dim3(256),
+  static_assert(sg_decode_smem(64) <= 48 * 1024, "no opt-in needed up to 64 heads");
+  const size_t smem = sg_decode_smem(a.H);
+  hipLaunchKernelGGL((sigmoid_attention_decode_kernel<ND, CAP>), dim3(num_decode, parts), dim3(512),
                      smem, st, static_cast<const __bf16*>(q), static_cast<const __bf16*>(k),
                      static_cast<const __bf16*>(v), a);
 }
