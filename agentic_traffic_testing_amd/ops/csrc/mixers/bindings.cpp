@@ -307,7 +307,8 @@ void sigmoid_attention(at::Tensor out, const at::Tensor& q, const at::Tensor& k_
                        const at::Tensor& tile_seq, const at::Tensor& tile_qoff, double scale,
                        double cap, const at::Tensor& bias, const at::Tensor& talk,
                        int64_t num_decode, int64_t max_decode_kv,
-                       const c10::optional<at::Tensor>& part, bool use_mfma) {
+                       const c10::optional<at::Tensor>& part, bool use_mfma,
+                       const c10::optional<at::Tensor>& split_out) {
   TORCH_CHECK(q.is_cuda() && q.dim() == 3 && q.is_contiguous() && out.is_cuda() &&
                   out.dim() == 3 && out.is_contiguous() && k_cache.dim() == 4 &&
                   v_cache.dim() == 4 && k_cache.is_contiguous() && v_cache.is_contiguous(),
@@ -343,6 +344,13 @@ void sigmoid_attention(at::Tensor out, const at::Tensor& q, const at::Tensor& k_
     part_ptr = part->data_ptr<float>();
     max_parts = part->size(2);
   }
+  if (split_out) {
+    f32c(*split_out, "split_out");
+    TORCH_CHECK(split_out->dim() == 4 && split_out->size(0) >= 1 && split_out->size(0) <= 64 &&
+                    split_out->size(1) == q.size(0) && split_out->size(2) == H &&
+                    split_out->size(3) == vdim,
+                "sigmoid_attention: split_out [shares, T, H, vdim]");
+  }
   const at::DeviceGuard g(q.device());
   rc_ok(mixk_sigmoid_attention(
             out.data_ptr(), q.data_ptr(), k_cache.data_ptr(), v_cache.data_ptr(),
@@ -350,7 +358,8 @@ void sigmoid_attention(at::Tensor out, const at::Tensor& q, const at::Tensor& k_
             seq_qstart.data_ptr<int>(), tile_seq.data_ptr<int>(), tile_qoff.data_ptr<int>(),
             tile_seq.numel(), num_decode, max_decode_kv, part_ptr, max_parts, H, G, dim, vdim, BS,
             static_cast<float>(scale), static_cast<float>(cap), bias.data_ptr<float>(),
-            talk.data_ptr<float>(), use_mfma, code(q), cur_stream()),
+            talk.data_ptr<float>(), split_out ? split_out->data_ptr<float>() : nullptr,
+            split_out ? split_out->size(0) : 1, q.size(0), use_mfma, code(q), cur_stream()),
         "sigmoid_attention");
 }
 
@@ -915,7 +924,7 @@ TORCH_LIBRARY(atta_mix, m) {
   m.def("sigmoid_attention(Tensor(a!) out, Tensor q, Tensor k_cache, Tensor v_cache, "
         "Tensor block_tables, Tensor seq_kvlen, Tensor seq_qstart, Tensor tile_seq, "
         "Tensor tile_qoff, float scale, float cap, Tensor bias, Tensor talk, int num_decode, "
-        "int max_decode_kv, Tensor? part, bool use_mfma) -> ()");
+        "int max_decode_kv, Tensor? part, bool use_mfma, Tensor? split_out) -> ()");
   m.def("short_conv_silu(Tensor(a!) out, Tensor x, Tensor w, Tensor(b!) conv_state, "
         "Tensor positions, Tensor seq_qstart, Tensor seq_slot, Tensor? bias) -> ()");
   m.def("gated_delta_rule(Tensor(a!) out, Tensor qkv, Tensor beta, Tensor decay, Tensor a_log, "

@@ -45,7 +45,8 @@ int mixk_sigmoid_attention(void* out, const void* q, const void* k_cache, const 
                            int num_tiles, int num_decode, int max_decode_kv, float* part,
                            int max_parts, int H, int G, int dim, int vdim, int block_size,
                            float scale, float cap, const float* bias, const float* talk,
-                           int use_mfma, int dtype, hipStream_t st);
+                           float* split_out, int split, int total_rows, int use_mfma, int dtype,
+                           hipStream_t st);
 int mixk_short_conv_silu(void* out, const void* x, int64_t x_stride, const void* w,
                          const void* bias, void* conv_state, const int* positions, const int* seq_qstart,
                          const int* seq_slot, int T, int S, int C, int taps, int dtype,

@@ -10,12 +10,12 @@
 // * matrix-core prefill kernel (bf16, dim % 8 == 0, vdim % 16 == 0, both <= 128, H <= 32): eight
 //   waves, 16 query tokens, 32-key tiles; wave w owns HW = ceil(H / 8) consecutive heads, whose
 //   Q fragments and O^T accumulators stay in its registers.  A head sits in slot
-//   4 (h / HW) + h % HW of 32 slots, so a wave's heads are always one 8-byte run and any H <= 32
-//   is one K = 32 step of the mixing product.  Per tile:
+//   SL (h / HW) + h % HW of 8 SL slots (SL = 2 up to 16 heads, else 4), so a wave's heads are always
+//   one run and any H is one K = 16 or 32 step of the mixing product.  Per tile:
 //     A  S^T[16 keys x 16 tokens] = K . Q^T (mfma 16x16x32, K rows straight from the pages), the
 //        weights in fp32, stored to LDS as an exact-to-2^-17 pair of bf16 (high + low part) in a
 //        [key][token][slot] image;
-//     B  mixed[16 keys x 16 heads] = W[16 keys x 32 slots] . talk^T per token (two products, high
+//     B  mixed[16 keys x 16 heads] = W[16 keys x slots] . talk^T per token (two products, high
 //        and low part, fp32 accumulation; talk holds bf16 checkpoint values), stored as bf16
 //        [slot][token][key];
 //     C  O^T[16 channels x 16 tokens] += V^T . mixed^T (V^T rows straight from the pages).
@@ -23,6 +23,8 @@
 //   barrier interval, so a tile costs two barriers (which order LDS only: the V fragments of the
 //   tile are in flight during B, the first K fragments of the next one during C).  The LDS
 //   images are XOR-swizzled (sg_place) so that no access of any phase has a bank conflict.
+//   A launch with few query tiles is split over the keys: every share writes fp32 partial rows, a
+//   join kernel adds them.
 // * matrix-core decode kernel (bf16, dim % 8 == 0, dim <= 256, vdim % 16 == 0, H <= 64): one
 //   workgroup per (sequence, 64-key partition), columns = the query heads of a KV head; the mix
 //   runs on the VALU in fp32; the partition's sums go to `part`, a combine kernel adds them.
@@ -42,8 +44,9 @@ constexpr int kSgTile = 64;     // query tokens per entry of the host's tile lis
 constexpr int kSgTok = 16;      // query tokens per workgroup (matrix-core prefill)
 constexpr int kSgKeys = 32;     // keys per tile
 constexpr int kSgPart = 64;     // keys per decode partition
-constexpr int kSgSlots = 32;    // head slots
-constexpr int kSgRow = kSgTok * 32;       // LDS row (of a key, of a slot): 16 tokens x 32 bf16
+constexpr int kSgRow = kSgTok * 32;   // LDS row of a slot: 16 tokens x 32 keys
+// head slots per wave (a run of 2 or 4, so 16 or 32 slots: the K of the mixing product)
+__host__ __device__ constexpr int sg_slots(int HW) { return HW <= 2 ? 2 : 4; }
 constexpr int kSgAcc = 64;      // accumulators per thread of the rows kernel
 // heads per wave whose Q fragments live in LDS: the widest form is short of registers (it uses
 // all of a CU's 160 KB)
@@ -61,6 +64,8 @@ struct SigArgs {
   const float* talk;    // [H, H]
   int bt_width, H, G, dim, vdim, block_size, bs_shift, max_parts, rows;
   float scale, cap;
+  float* split_out;     // prefill split over the keys: fp32 partial rows [split, T, H, vdim]
+  int split, total_rows;
 };
 
 // Weight of one key on the fast transcendental units.  With a cap: t = tanh(y) as
@@ -86,12 +91,13 @@ __device__ __forceinline__ sg_bf16x8 zero_frag() {
   const sg_u32x4 z = {0u, 0u, 0u, 0u};
   return __builtin_bit_cast(sg_bf16x8, z);
 }
-// Place of (row, token, 16-byte chunk) in an LDS image of rows of 16 tokens x 4 chunks.  The token is
-// XORed with the row and the chunk with the token's place, so that neither 16 tokens of a row nor
-// 16 rows of a token share a bank.
+// Place of (row, token, chunk) in an LDS image of rows of 16 tokens x 4 chunks of CH elements.  The
+// token is XORed with the row and the chunk with the token's place, so that neither 16 tokens of a
+// row nor 16 rows of a token share a bank.
+template <int CH>
 __device__ __forceinline__ int sg_place(int row, int t, int chunk) {
   const int p = t ^ (row & 15);
-  return row * kSgRow + p * 32 + ((chunk ^ (p >> 2)) << 3);
+  return row * (kSgTok * 4 * CH) + p * (4 * CH) + (chunk ^ (p >> 2)) * CH;
 }
 
 // A copy the compiler knows nothing about: what is computed from it stays inside the loop instead of
@@ -117,18 +123,29 @@ __device__ __forceinline__ void lds_barrier() {
 
 // ONE: the heads of a wave share one KV head (H / G is a multiple of HW), so its K and V fragments
 // are loaded once per tile, ahead of their use.
+// Forms with few heads fit twice on a CU.
+constexpr int sg_waves(int HW, int NV) { return HW * NV <= 8 ? 4 : 2; }
+
+// V fragments in flight: what the registers leave.
+constexpr int sg_v_flight(int HW, int NV) {
+  return HW * NV >= 32 ? NV / 4 : (HW * NV == 8 && NV == 8 ? NV / 2 : NV);
+}
+
 template <int HW, int ND, int NV, bool CAP, bool ONE>   // dim <= 32 ND, vdim <= 16 NV, H <= 8 HW
-__global__ void __launch_bounds__(512)
+__global__ void __launch_bounds__(512, sg_waves(HW, NV))
 sigmoid_attention_mfma_kernel(__bf16* __restrict__ out, const __bf16* __restrict__ q,
                               const __bf16* __restrict__ k_cache,
                               const __bf16* __restrict__ v_cache, SigArgs a) {
   constexpr int QL = sg_q_lds(HW, ND), QR = HW - QL;     // heads with Q in LDS / in registers
   constexpr int QS = 32 * ND;                            // LDS row of one token's Q
-  constexpr int NF = HW * NV >= 32 ? NV / 2 : NV;        // V fragments in flight (registers)
+  constexpr int NF = sg_v_flight(HW, NV);
   extern __shared__ __attribute__((aligned(16))) char sg_smem[];
-  __bf16* w_hi = reinterpret_cast<__bf16*>(sg_smem);     // [32 keys][kSgRow]
-  __bf16* w_lo = w_hi + kSgKeys * kSgRow;
-  __bf16* mixed = w_lo + kSgKeys * kSgRow;               // [32 slots][kSgRow]
+  constexpr int SL = sg_slots(HW), kSlots = 8 * SL, CH = 2 * SL;   // CH: slots per chunk
+  typedef __attribute__((ext_vector_type(SL))) __bf16 slots_t;           // a wave's slots
+  typedef __attribute__((ext_vector_type(CH))) __bf16 chunk_t;           // K fragment of the mix
+  __bf16* w_hi = reinterpret_cast<__bf16*>(sg_smem);     // [32 keys][16 tokens][kSlots]
+  __bf16* w_lo = w_hi + kSgKeys * kSgTok * kSlots;
+  __bf16* mixed = w_lo + kSgKeys * kSgTok * kSlots;      // [kSlots][16 tokens][32 keys]
   const int H = a.H, G = a.G, dim = a.dim, vdim = a.vdim, bs = a.block_size;
   const int rep = H / G, nv = vdim >> 4;
   // the tiles with the most keys come last in the list: start those first
@@ -140,13 +157,17 @@ sigmoid_attention_mfma_kernel(__bf16* __restrict__ out, const __bf16* __restrict
   const int ntok = min(kSgTok, n - qo);
   const int pos0 = kvlen - n + qo;          // position of the first query token
   const int kend = pos0 + ntok;             // keys [0, kend) are visible to somebody
+  // this workgroup's share of the key tiles
+  const int ntiles = (kend + kSgKeys - 1) / kSgKeys, per = (ntiles + a.split - 1) / a.split;
+  const int kfirst = static_cast<int>(blockIdx.y) * per * kSgKeys;
+  const int kstop = min(kend, kfirst + per * kSgKeys);
   const int tid = threadIdx.x, lane = tid & 63, r = lane & 15, c = lane >> 4;
   const int w = __builtin_amdgcn_readfirstlane(tid >> 6);
   const int h0 = w * HW;
   const bool wave_on = h0 < H;
   const int qpos = pos0 + r;
   // head QR + e of the wave in LDS: this lane's row of the e-th 16-token block, chunks XORed with r
-  __bf16* q_rows = mixed + kSgSlots * kSgRow + (w * QL * kSgTok + r) * QS;
+  __bf16* q_rows = mixed + kSlots * kSgRow + (w * QL * kSgTok + r) * QS;
   auto q_lds = [&](int e, int st, int rr) {
     return q_rows + e * kSgTok * QS + (((st * 4 + c) ^ (rr & (4 * ND - 1))) << 3);
   };
@@ -172,21 +193,30 @@ sigmoid_attention_mfma_kernel(__bf16* __restrict__ out, const __bf16* __restrict
   }
   const float k1 = CAP ? 2.0f * kLog2e * a.scale / a.cap : -kLog2e * a.scale;
   const float k2 = 2.0f * a.cap * kLog2e;
-  // B operand of the mix: column = output slot, rows = input slots 8 c .. 8 c + 7
-  sg_bf16x8 tf[2];
+  // B operand of the mix: column = output slot, rows = this lane's CH input slots
+  chunk_t tf[kSlots / 16];
 #pragma unroll
-  for (int ht = 0; ht < 2; ++ht) {
+  for (int ht = 0; ht < kSlots / 16; ++ht) {
     const int so = ht * 16 + r;
-    const int ho = (so >> 2) * HW + (so & 3);
+    const int ho = (so / SL) * HW + so % SL;
 #pragma unroll
-    for (int j = 0; j < 8; ++j) {
-      const int si = 8 * c + j;
-      const int hi = (si >> 2) * HW + (si & 3);
-      const bool ok = (so & 3) < HW && ho < H && (si & 3) < HW && hi < H;
+    for (int j = 0; j < CH; ++j) {
+      const int si = CH * c + j;
+      const int hi = (si / SL) * HW + si % SL;
+      const bool ok = so % SL < HW && ho < H && si % SL < HW && hi < H;
       tf[ht][j] = static_cast<__bf16>(ok ? a.talk[ho * H + hi] : 0.f);
     }
   }
-  const int nht = (H - 1) / HW >= 4 ? 2 : 1;   // output slot tiles in use
+  const int nht = ((H - 1) / HW * SL + HW + 15) / 16;   // output slot tiles in use
+  auto mix = [](chunk_t x, chunk_t t, sg_f32x4 d) {
+    if constexpr (SL == 4) {
+      return __builtin_amdgcn_mfma_f32_16x16x32_bf16(x, t, d, 0, 0, 0);
+    } else {
+      typedef __attribute__((ext_vector_type(4))) short s16x4;
+      return __builtin_amdgcn_mfma_f32_16x16x16bf16_1k(__builtin_bit_cast(s16x4, x),
+                                                       __builtin_bit_cast(s16x4, t), d, 0, 0, 0);
+    }
+  };
   sg_f32x4 O[HW][NV];
 #pragma unroll
   for (int hh = 0; hh < HW; ++hh)
@@ -228,9 +258,9 @@ sigmoid_attention_mfma_kernel(__bf16* __restrict__ out, const __bf16* __restrict
     const int rr = fresh(r);
 #pragma unroll
     for (int i = 0; i < 4; ++i) {
-      sg_bf16x4 hi, lo;
+      slots_t hi, lo;
 #pragma unroll
-      for (int hh = 0; hh < 4; ++hh) {
+      for (int hh = 0; hh < SL; ++hh) {
         float x = 0.f;
         if (hh < HW) {
           x = sig_weight<CAP>(S[hh < HW ? hh : 0][i], k1, k2, k3[hh < HW ? hh : 0]);
@@ -239,9 +269,9 @@ sigmoid_attention_mfma_kernel(__bf16* __restrict__ out, const __bf16* __restrict
         hi[hh] = static_cast<__bf16>(x);
         lo[hh] = static_cast<__bf16>(x - static_cast<float>(hi[hh]));
       }
-      const int o = sg_place(sub * 16 + 4 * c + i, rr, w >> 1) + (w & 1) * 4;
-      *reinterpret_cast<sg_bf16x4*>(w_hi + o) = hi;
-      *reinterpret_cast<sg_bf16x4*>(w_lo + o) = lo;
+      const int o = sg_place<CH>(sub * 16 + 4 * c + i, rr, w >> 1) + (w & 1) * SL;
+      *reinterpret_cast<slots_t*>(w_hi + o) = hi;
+      *reinterpret_cast<slots_t*>(w_lo + o) = lo;
     }
   };
 
@@ -277,22 +307,24 @@ sigmoid_attention_mfma_kernel(__bf16* __restrict__ out, const __bf16* __restrict
     }
   };
 
-  int pk0 = page_at(r), pk1 = page_at(16 + r), pv = page_at(8 * c);
+  // (a share without keys runs the prologue on clamped addresses and stores zeros)
+  int pk0 = page_at(kfirst + r), pk1 = page_at(kfirst + 16 + r), pv = page_at(kfirst + 8 * c);
   if (wave_on) {
-    if (ONE) load_k(ka, pk0, r, g0);
-    scores(0, pk0, pk1);
+    if (ONE) load_k(ka, pk0, kfirst + r, g0);
+    scores(kfirst, pk0, pk1);
   } else {   // this wave's slots never hold a head: zero them once
-    const sg_bf16x4 z = {static_cast<__bf16>(0.f), static_cast<__bf16>(0.f),
-                         static_cast<__bf16>(0.f), static_cast<__bf16>(0.f)};
+    slots_t z;
+#pragma unroll
+    for (int hh = 0; hh < SL; ++hh) z[hh] = static_cast<__bf16>(0.f);
     for (int key = c; key < kSgKeys; key += 4) {
-      const int o = sg_place(key, r, w >> 1) + (w & 1) * 4;
-      *reinterpret_cast<sg_bf16x4*>(w_hi + o) = z;
-      *reinterpret_cast<sg_bf16x4*>(w_lo + o) = z;
+      const int o = sg_place<CH>(key, r, w >> 1) + (w & 1) * SL;
+      *reinterpret_cast<slots_t*>(w_hi + o) = z;
+      *reinterpret_cast<slots_t*>(w_lo + o) = z;
     }
   }
-  pk0 = page_at(kSgKeys + r);
-  pk1 = page_at(kSgKeys + 16 + r);
-  for (int k0 = 0; k0 < kend; k0 += kSgKeys) {
+  pk0 = page_at(kfirst + kSgKeys + r);
+  pk1 = page_at(kfirst + kSgKeys + 16 + r);
+  for (int k0 = kfirst; k0 < kstop; k0 += kSgKeys) {
     const int nk = k0 + kSgKeys, t8 = k0 + 8 * c;
     const __bf16* vb = v_cache + pv * vpage + (min(t8, last) & bmask & ~7) + static_cast<int64_t>(r) * bs;
     sg_bf16x8 vf[NF];
@@ -311,18 +343,19 @@ sigmoid_attention_mfma_kernel(__bf16* __restrict__ out, const __bf16* __restrict
       const int t = 2 * w + tt;
 #pragma unroll
       for (int half = 0; half < 2; ++half) {
-        const int o = sg_place(half * 16 + rb, t, c);
-        const sg_bf16x8 ah = ld_frag(w_hi + o), al = ld_frag(w_lo + o);
+        const int o = sg_place<CH>(half * 16 + rb, t, c);
+        const chunk_t ah = *reinterpret_cast<const chunk_t*>(w_hi + o);
+        const chunk_t al = *reinterpret_cast<const chunk_t*>(w_lo + o);
 #pragma unroll
-        for (int ht = 0; ht < 2; ++ht) {
+        for (int ht = 0; ht < kSlots / 16; ++ht) {
           if (ht < nht) {
             sg_f32x4 D = {0.f, 0.f, 0.f, 0.f};
-            D = __builtin_amdgcn_mfma_f32_16x16x32_bf16(al, tf[ht], D, 0, 0, 0);
-            D = __builtin_amdgcn_mfma_f32_16x16x32_bf16(ah, tf[ht], D, 0, 0, 0);
+            D = mix(al, tf[ht], D);
+            D = mix(ah, tf[ht], D);
             sg_bf16x4 e;
 #pragma unroll
             for (int i = 0; i < 4; ++i) e[i] = static_cast<__bf16>(D[i]);
-            *reinterpret_cast<sg_bf16x4*>(mixed + sg_place(ht * 16 + rb, t, half * 2 + (c >> 1)) +
+            *reinterpret_cast<sg_bf16x4*>(mixed + sg_place<8>(ht * 16 + rb, t, half * 2 + (c >> 1)) +
                                           (c & 1) * 4) = e;
           }
         }
@@ -343,7 +376,7 @@ sigmoid_attention_mfma_kernel(__bf16* __restrict__ out, const __bf16* __restrict
           }
 #pragma unroll
           for (int hh = 0; hh < HW; ++hh) {
-            const sg_bf16x8 pf = ld_frag(mixed + sg_place(4 * w + hh, rc, c));
+            const sg_bf16x8 pf = ld_frag(mixed + sg_place<8>(SL * w + hh, rc, c));
 #pragma unroll
             for (int e = 0; e < NF; ++e)
               O[hh][vt0 + e] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(vf[e], pf, O[hh][vt0 + e], 0, 0, 0);
@@ -355,7 +388,7 @@ sigmoid_attention_mfma_kernel(__bf16* __restrict__ out, const __bf16* __restrict
       } else {
 #pragma unroll
         for (int hh = 0; hh < HW; ++hh) {
-          const sg_bf16x8 pf = ld_frag(mixed + sg_place(4 * w + hh, rc, c));
+          const sg_bf16x8 pf = ld_frag(mixed + sg_place<8>(SL * w + hh, rc, c));
           const __bf16* vh = vb + static_cast<int64_t>(kv_head(hh)) * vdim * bs;
           sg_bf16x8 vg[NV];
 #pragma unroll
@@ -369,7 +402,7 @@ sigmoid_attention_mfma_kernel(__bf16* __restrict__ out, const __bf16* __restrict
             O[hh][vt] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(vg[vt], pf, O[hh][vt], 0, 0, 0);
         }
       }
-      if (nk < kend) scores(nk, pk0, pk1);
+      if (nk < kstop) scores(nk, pk0, pk1);
     }
     pk0 = page_at(nk + kSgKeys + r);
     pk1 = page_at(nk + kSgKeys + 16 + r);
@@ -379,6 +412,13 @@ sigmoid_attention_mfma_kernel(__bf16* __restrict__ out, const __bf16* __restrict
   for (int hh = 0; hh < HW; ++hh) {
     const int h = h0 + hh;
     if (h < H) {
+      if (a.split > 1) {
+        float* o = a.split_out + ((static_cast<int64_t>(blockIdx.y) * a.total_rows + row0 + qo + r) * H + h) * vdim + 4 * c;
+#pragma unroll
+        for (int vt = 0; vt < NV; ++vt)
+          if (vt < nv) *reinterpret_cast<sg_f32x4*>(o + vt * 16) = O[hh][vt];
+        continue;
+      }
       __bf16* o = out + (static_cast<int64_t>(row0 + qo + r) * H + h) * vdim + 4 * c;
 #pragma unroll
       for (int vt = 0; vt < NV; ++vt) {
@@ -390,6 +430,25 @@ sigmoid_attention_mfma_kernel(__bf16* __restrict__ out, const __bf16* __restrict
         }
       }
     }
+  }
+}
+
+// Rows of the tile list: the sum of the key shares' partial rows.
+__global__ void sigmoid_attention_join_kernel(__bf16* __restrict__ out, SigArgs a) {
+  const int s = a.tile_seq[blockIdx.x], qo = a.tile_qoff[blockIdx.x] + blockIdx.y;
+  const int row0 = a.seq_qstart[s], n = a.seq_qstart[s + 1] - row0;
+  if (qo >= n || a.seq_kvlen[s] <= 0) return;
+  const int width = a.H * a.vdim;   // a multiple of 16
+  const int64_t base = static_cast<int64_t>(row0 + qo) * width;
+  for (int i = threadIdx.x * 8; i < width; i += blockDim.x * 8) {
+    float v[8] = {0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f};
+    for (int z = 0; z < a.split; ++z) {
+      float p[8];
+      ld8(a.split_out + static_cast<int64_t>(z) * a.total_rows * width + base + i, p);
+#pragma unroll
+      for (int e = 0; e < 8; ++e) v[e] += p[e];
+    }
+    st8(out + base + i, v);
   }
 }
 
@@ -632,18 +691,21 @@ int sg_smem_opt_in(K kernel, size_t smem) {
 template <int HW, int ND, int NV, bool CAP, bool ONE>
 int sg_launch_prefill(void* out, const void* q, const void* k, const void* v, const SigArgs& a,
                       int num_tiles, hipStream_t st) {
-  const size_t smem = sizeof(__bf16) * ((2 * kSgKeys + kSgSlots) * kSgRow +
-                                        sg_q_lds(HW, ND) * 8 * kSgTok * 32 * ND);
-  static_assert(sizeof(__bf16) * (3 * 32 * 512 + 2 * 8 * 16 * 128) == 160 * 1024, "all of the LDS");
+  constexpr size_t smem = sizeof(__bf16) * (3 * kSgKeys * kSgTok * 8 * sg_slots(HW) +
+                                            sg_q_lds(HW, ND) * 8 * kSgTok * 32 * ND);
+  static_assert(smem <= 160 * 1024, "LDS of a CU");
   static bool opted = false;
   if (!opted) {
     if (int rc = sg_smem_opt_in(sigmoid_attention_mfma_kernel<HW, ND, NV, CAP, ONE>, smem)) return rc;
     opted = true;
   }
   hipLaunchKernelGGL((sigmoid_attention_mfma_kernel<HW, ND, NV, CAP, ONE>),
-                     dim3(num_tiles * (kSgTile / kSgTok)), dim3(512), smem, st,
+                     dim3(num_tiles * (kSgTile / kSgTok), a.split), dim3(512), smem, st,
                      static_cast<__bf16*>(out), static_cast<const __bf16*>(q),
                      static_cast<const __bf16*>(k), static_cast<const __bf16*>(v), a);
+  if (a.split > 1)
+    hipLaunchKernelGGL(sigmoid_attention_join_kernel, dim3(num_tiles, kSgTile), dim3(256), 0, st,
+                       static_cast<__bf16*>(out), a);
   return static_cast<int>(hipGetLastError());
 }
 
@@ -729,15 +791,17 @@ extern "C" int mixk_sigmoid_attention(void* out, const void* q, const void* k_ca
                                       int num_decode, int max_decode_kv, float* part,
                                       int max_parts, int H, int G, int dim, int vdim,
                                       int block_size, float scale, float cap, const float* bias,
-                                      const float* talk, int use_mfma, int dtype, hipStream_t st) {
+                                      const float* talk, float* split_out, int split,
+                                      int total_rows, int use_mfma, int dtype, hipStream_t st) {
   if (num_tiles <= 0 && num_decode <= 0) return 0;
-  if (G <= 0 || H % G != 0 || cap < 0.f) return -1;
+  if (G <= 0 || H % G != 0 || cap < 0.f || split < 1) return -1;
   const int parts = (max_decode_kv + kSgPart - 1) / kSgPart;
   if (num_decode > 0 && (parts < 1 || parts > max_parts || part == nullptr)) return -1;
   int bs_shift = 0;
   while ((1 << bs_shift) < block_size) ++bs_shift;
   const SigArgs a{block_tables, seq_kvlen, seq_qstart, tile_seq, tile_qoff, part, bias, talk,
-                  bt_width, H, G, dim, vdim, block_size, bs_shift, max_parts, 0, scale, cap};
+                  bt_width, H, G, dim, vdim, block_size, bs_shift, max_parts, 0, scale, cap,
+                  split_out, split_out != nullptr ? split : 1, total_rows};
   const bool pages_ok = block_size >= 8 && (block_size & (block_size - 1)) == 0;
   const bool base_ok = use_mfma && dtype == 0 && pages_ok && dim % 8 == 0 && vdim % 16 == 0;
   int rc = 0, rows_tiles = num_tiles, rows_decode = num_decode;

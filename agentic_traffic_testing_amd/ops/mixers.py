@@ -75,6 +75,7 @@ def _native():
 ATTN_TILE_TOKENS = 64     # query tokens per prefill attention tile (the block manager tiles by it)
 DECODE_PART_TOKENS = 128  # keys per decode-attention partition
 SIGMOID_PART_TOKENS = 64  # ... of the sigmoid attention
+SIGMOID_MAX_SPLIT = int(os.environ.get("ATTA_MIX_SIGMOID_SPLIT", "4"))  # key shares of a tile
 ATTENTION_MFMA = os.environ.get("ATTA_MIX_ATTENTION_MFMA", "1") != "0"
 ACT_SILU, ACT_SIGMOID, ACT_GELU_TANH = 0, 1, 2
 _SCORE_CODES = {"sigmoid": 0, "softmax": 1, "logit": 2}
@@ -249,10 +250,18 @@ def sigmoid_attention(q, k_cache, v_cache, block_tables, seq_kvlen, seq_qstart, 
         parts = max(1, -(-int(max_decode_kv) // SIGMOID_PART_TOKENS))
         part = torch.empty(num_decode, q.shape[1], parts, v_cache.shape[2], dtype=torch.float32,
                            device=q.device)
+    # few query tiles: the key range is cut over `split` workgroups per tile so the launch fills the
+    # chip; the fp32 partial rows are added by a second kernel
+    split_out, tiles = None, 4 * tile_seq.shape[0]
+    split = min(SIGMOID_MAX_SPLIT, 512 // tiles) if tiles else 1
+    if split > 1 and q.dtype == torch.bfloat16 and ATTENTION_MFMA:
+        split_out = torch.empty(split, q.shape[0], q.shape[1], v_cache.shape[2],
+                                dtype=torch.float32, device=q.device)
     if tile_seq.shape[0] > 0 or num_decode > 0:
         _native().sigmoid_attention(out, q, k_cache, v_cache, block_tables, seq_kvlen, seq_qstart,
                                     tile_seq, tile_qoff, float(scale), float(softcap), bias, talk,
-                                    num_decode, max(1, int(max_decode_kv)), part, ATTENTION_MFMA)
+                                    num_decode, max(1, int(max_decode_kv)), part, ATTENTION_MFMA,
+                                    split_out)
     return out
 
 

@@ -747,7 +747,7 @@ def ragged_pages(md, G, dim, vdim, bs, dt, seed=0):
     (24, 8, 128, 96, 8, 15.0), (32, 8, 128, 128, 16, 30.0), (3, 1, 16, 16, 16, 5.0),
     (20, 2, 72, 32, 16, 9.0), (5, 5, 13, 9, 16, 4.0), (40, 8, 32, 16, 16, 6.0),
     (4, 2, 32, 32, 12, 6.0), (8, 8, 192, 160, 16, 11.0), (1, 1, 8, 16, 16, 0.0)])
-def test_sigmoid_attention(dt, H, G, dim, vdim, bs, cap):
+def test_sigmoid_attention(dt, H, G, dim, vdim, bs, cap, monkeypatch):
     torch.manual_seed(1)
     lens, starts = [1, 1, 37, 2, 150, 64, 16], [0, 170, 0, 131, 45, 200, 15]
     md = ragged(lens, starts, list(range(7)), bs=bs, width=48)
@@ -760,7 +760,9 @@ def test_sigmoid_attention(dt, H, G, dim, vdim, bs, cap):
     want = mref.sigmoid_attention(q, kc, vc, md["block_tables"], md["seq_kvlen"],
                                   md["seq_qstart"], scale, cap, bias, talk).float()
     g = cuda(md)
-    for nd in (0, 2):   # the single-row portions in the tile kernel, then as decode rows
+    # the single-row portions in the tile kernel, then as decode rows; with and without key shares
+    for nd, shares in ((0, 4), (2, 4), (2, 1), (0, 7)):
+        monkeypatch.setattr(mx, "SIGMOID_MAX_SPLIT", shares)
         keep = md["tile_seq"] >= nd
         got = mx.sigmoid_attention(q.cuda(), kc.cuda(), vc.cuda(), g["block_tables"],
                                    g["seq_kvlen"], g["seq_qstart"],
