@@ -21,8 +21,8 @@
 //     C  O^T[16 channels x 16 tokens] += V^T . mixed^T (V^T rows straight from the pages).
 //   B needs A of all waves and C needs B of all waves; C of a tile and A of the next share one
 //   barrier interval, so a tile costs two barriers (which order LDS only: the V fragments of the
-//   tile are in flight during B, the first K fragments of the next one during C).  The LDS
-//   images are XOR-swizzled (sg_place) so that no access of any phase has a bank conflict.
+//   tile are in flight during B, the first K fragments of the next one late in C).  The LDS images
+//   are XOR-swizzled (sg_place) to spread the accesses of every phase over the banks.
 //   A launch with few query tiles is split over the keys: every share writes fp32 partial rows, a
 //   join kernel adds them.
 // * matrix-core decode kernel (bf16, dim % 8 == 0, dim <= 256, vdim % 16 == 0, H <= 64): one
@@ -392,7 +392,8 @@ sigmoid_attention_mfma_kernel(__bf16* __restrict__ out, const __bf16* __restrict
           const __bf16* vh = vb + static_cast<int64_t>(kv_head(hh)) * vdim * bs;
           sg_bf16x8 vg[NV];
 #pragma unroll
-          for (int vt = 0; vt < NV; ++vt) vg[vt] = ld_frag(vh + static_cast<int64_t>(min(vt, nv - 1)) * 16 * bs);
+          for (int vt = 0; vt < NV; ++vt)
+            vg[vt] = ld_frag(vh + static_cast<int64_t>(min(vt, nv - 1)) * 16 * bs);
           if (tail) {
 #pragma unroll
             for (int vt = 0; vt < NV; ++vt) vg[vt] = keep_keys(vg[vt], t8, kend);
@@ -413,7 +414,8 @@ sigmoid_attention_mfma_kernel(__bf16* __restrict__ out, const __bf16* __restrict
     const int h = h0 + hh;
     if (h < H) {
       if (a.split > 1) {
-        float* o = a.split_out + ((static_cast<int64_t>(blockIdx.y) * a.total_rows + row0 + qo + r) * H + h) * vdim + 4 * c;
+        const int64_t row = static_cast<int64_t>(blockIdx.y) * a.total_rows + row0 + qo + r;
+        float* o = a.split_out + (row * H + h) * vdim + 4 * c;
 #pragma unroll
         for (int vt = 0; vt < NV; ++vt)
           if (vt < nv) *reinterpret_cast<sg_f32x4*>(o + vt * 16) = O[hh][vt];

@@ -559,8 +559,9 @@ def _moe_experts_library(h, idx, wts, w_gu, w_down, limit, alpha, silu_glu=False
 def moe_route(logits, top, score="sigmoid", correction=None, groups=1, keep=1, renorm=False):
     """fp32 router logits [T, E] -> (expert index int32 [T, top], score fp32 [T, top]) of every
     row's ``top`` largest scores (ties: lowest index).  ``score``: "sigmoid", "softmax" over
-    the row, or "logit" (the logits choose, the weights are their softmax over the chosen ones).  ``correction`` fp32 [E] is added to the scores for the choice only (the returned
-    weights are the plain scores).  ``groups`` > 1: the experts form that many equal runs of
+    the row, or "logit" (the logits choose, the weights are their softmax over the chosen ones).
+    ``correction`` fp32 [E] is added to the scores for the choice only (the returned weights are
+    the plain scores).  ``groups`` > 1: the experts form that many equal runs of
     neighbours, a group's score is its largest choice score, and only experts of the ``keep``
     best groups can be chosen.  ``renorm``: the chosen scores are divided by their sum + 1e-20."""
     E = logits.shape[1]
