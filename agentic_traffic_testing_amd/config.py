@@ -306,7 +306,7 @@ class LatentAttentionConfig:
     rot_base: float
     scale: float
     kv_from: int = -1
-    window: int = 0   # sliding window (Kolotar); 0: every earlier key
+    window: int = 0   # sliding window; 0: every earlier key
 
 
 @dataclass(frozen=True)
@@ -962,6 +962,207 @@ HYBRID_PRESETS.update({
                                        192, 1024),
 })
 ARCHITECTURES["Kolotar"] = KolotarConfig.from_dict
+
+
+# ---------------------------------------------------------------------------------------
+# Tofodra: decoder with an RMS norm before and after every sub-layer and a per-channel scale on the
+# branches; a layer's mixer is retention (linear attention with a fixed decay per head),
+# differential attention inside a sliding window that keeps the first tokens, or latent attention
+# with an optionally shared cache; its feed-forward is a dense clamped GLU or routed SiLU-GLU
+# experts with a shared one.
+
+@dataclass(frozen=True)
+class RetentionConfig:
+    """Linear attention without a denominator: per head S <- decay S + k v^T, o = S^T q, rotate-half
+    positions on the first ``rot_dims`` channels of q and k, k times dim^-0.5; each head's output
+    divided by its root mean square, then a SiLU gate over all channels."""
+    heads: int
+    dim: int
+    vdim: int
+    decay: tuple = ()
+    rot_dims: int = 0
+    rot_base: float = 10000.0
+
+
+@dataclass(frozen=True)
+class DifferentialAttentionConfig:
+    """Grouped-query attention of two softmax maps over the same values, o = a1 - lambda a2 with one
+    learned lambda per layer, divided by its root mean square per head and times 1 - ``diff``;
+    biased q / k / v projections, no rotation, a sliding window of ``window`` keys (0: all earlier
+    keys) beside the sequence's first ``keep_first`` tokens, element-wise sigmoid output gate."""
+    heads: int
+    kv_heads: int
+    dim: int
+    vdim: int
+    scale: float
+    diff: float
+    window: int = 0
+    keep_first: int = 0
+
+
+@dataclass(frozen=True)
+class ScaledMoeConfig:
+    """``experts`` SiLU-GLU feed-forward layers of width ``ff``; a token runs the ``top`` with the
+    largest sigmoid router scores, weighted by those scores normalised to sum ``scale``.  A shared
+    expert of width ``shared_ff`` (0: none) runs for every token."""
+    experts: int
+    top: int
+    ff: int
+    scale: float = 1.0
+    shared_ff: int = 0
+
+
+@dataclass(frozen=True)
+class TofodraLayerConfig:
+    kind: str                 # "retention" | "attention" | "latent_attention"
+    mixer: object = None
+    ff: int = 0               # dense clamped-GLU width (0: none, or see ``moe``)
+    limit: float = 0.0        # clamp of the dense GLU
+    moe: ScaledMoeConfig | None = None
+
+
+@dataclass(frozen=True)
+class TofodraConfig:
+    name: str = "tofodra"
+    vocab_size: int = 1024
+    hidden_size: int = 256
+    layers: tuple = ()
+    rms_norm_eps: float = 1e-5
+    embed_scale: float = 1.0
+    bos_token_id: int = 0
+    eos_token_ids: tuple = ()
+    max_position_embeddings: int = 1 << 20
+    family: str = "tofodra"
+
+    @property
+    def num_layers(self) -> int:
+        return len(self.layers)
+
+    @staticmethod
+    def from_dict(c: dict, name: str = "tofodra") -> "TofodraConfig":
+        """Parse the checkpoint's config.json (keys: vocab, width, norm.eps, embedding.scale,
+        layers[].{type, mixer, mlp}; retention: heads, dim, vdim, decay, rot.{dims, base};
+        attention: heads, kv_heads, dim, vdim, scale, diff, mask.{size, keep_first};
+        latent_attention: heads, dim, rot_dim, vdim, kv_rank, scale, rot.{dims, base}, kv_from; mlp:
+        kind dense {ff, limit} or moe {expert.ff, router.{experts, top, scale}, shared.ff}, or
+        null).  An absent rot, mask, kv_from, embedding or shared means none."""
+
+        def rotary(m, width, i, dims=0):
+            rot = m.get("rot") or {}
+            dims, base = int(rot.get("dims", dims)), float(rot.get("base", 10000.0))
+            if dims % 2 or not 0 <= dims <= width:
+                raise ValueError(f"layer {i}: rot.dims must be even and <= {width}")
+            return dims, base
+
+        layers = []
+        for i, L in enumerate(c["layers"]):
+            m, t = L["mixer"], L["type"]
+            if t == "retention":
+                dims, base = rotary(m, int(m["dim"]), i)
+                mc = RetentionConfig(heads=int(m["heads"]), dim=int(m["dim"]),
+                                     vdim=int(m.get("vdim", m["dim"])),
+                                     decay=tuple(float(d) for d in m["decay"]), rot_dims=dims,
+                                     rot_base=base)
+                if len(mc.decay) != mc.heads:
+                    raise ValueError(f"layer {i}: one decay per head")
+            elif t == "attention":
+                mask = m.get("mask") or {}
+                mc = DifferentialAttentionConfig(
+                    heads=int(m["heads"]), kv_heads=int(m.get("kv_heads", m["heads"])),
+                    dim=int(m["dim"]), vdim=int(m.get("vdim", m["dim"])), scale=float(m["scale"]),
+                    diff=float(m["diff"]), window=int(mask.get("size") or 0),
+                    keep_first=int(mask.get("keep_first") or 0))
+                if mc.kv_heads < 1 or mc.heads % mc.kv_heads:
+                    raise ValueError(f"layer {i}: heads must be a multiple of kv_heads")
+                if mc.window < 0 or mc.keep_first < 0:
+                    raise ValueError(f"layer {i}: mask sizes must not be negative")
+            elif t == "latent_attention":
+                dims, base = rotary(m, int(m["rot_dim"]), i, int(m["rot_dim"]))
+                mc = LatentAttentionConfig(
+                    heads=int(m["heads"]), dim=int(m["dim"]), rot_dim=int(m["rot_dim"]),
+                    vdim=int(m["vdim"]), kv_rank=int(m["kv_rank"]), q_rank=0, rot_dims=dims,
+                    rot_base=base, scale=float(m["scale"]),
+                    kv_from=-1 if m.get("kv_from") is None else int(m["kv_from"]))
+                if mc.kv_from >= 0:
+                    src = layers[mc.kv_from].mixer if mc.kv_from < i else None
+                    if not isinstance(src, LatentAttentionConfig) or src.kv_from >= 0 or \
+                            (src.kv_rank, src.rot_dim, src.rot_dims, src.rot_base) != \
+                            (mc.kv_rank, mc.rot_dim, mc.rot_dims, mc.rot_base):
+                        raise ValueError(f"layer {i}: kv_from must name an earlier latent-attention "
+                                         "layer with its own cache and the same latent geometry")
+            else:
+                raise ValueError(f"unknown layer type {t!r}")
+            mlp, kw = L.get("mlp"), {}
+            if mlp:
+                kind = str(mlp.get("kind", "dense"))
+                if kind == "dense":
+                    kw = {"ff": int(mlp["ff"]), "limit": float(mlp["limit"])}
+                elif kind == "moe":
+                    r = mlp["router"]
+                    moe = ScaledMoeConfig(
+                        experts=int(r["experts"]), top=int(r["top"]), ff=int(mlp["expert"]["ff"]),
+                        scale=float(r.get("scale", 1.0)),
+                        shared_ff=int((mlp.get("shared") or {}).get("ff", 0)))
+                    if not 1 <= moe.top <= moe.experts:
+                        raise ValueError(f"layer {i}: router.top must be in [1, experts]")
+                    kw = {"moe": moe}
+                else:
+                    raise ValueError(f"unsupported feed-forward kind {kind!r}")
+            layers.append(TofodraLayerConfig(t, mc, **kw))
+        return TofodraConfig(name=name, vocab_size=int(c["vocab"]), hidden_size=int(c["width"]),
+                             layers=tuple(layers), rms_norm_eps=float(c["norm"]["eps"]),
+                             embed_scale=float((c.get("embedding") or {}).get("scale", 1.0)))
+
+
+def tofodra_preset(name: str, vocab: int, width: int, ff: int, pattern: str, heads: int,
+                   kv_heads: int, dim: int, kv_rank: int, window: int, experts: int = 8,
+                   top: int = 2, expert_ff: int = 0, rot_dim: int = 64,
+                   shared_ff: int = 0) -> TofodraConfig:
+    """A Tofodra shape for benchmarks and tests: two letters per layer, mixer (``r`` retention,
+    ``a`` differential attention, ``l`` latent attention, ``s`` latent attention on the first ``l``
+    layer's cache) then feed-forward (``d`` dense, ``e`` experts, ``-`` none).  The two attention
+    maps split ``dim`` between them, so q, k and v are as wide as those of ``heads`` plain heads."""
+    ret = RetentionConfig(heads, dim, dim,
+                          tuple(1.0 - 2.0 ** (-5.0 - 7.0 * h / max(1, heads - 1))
+                                for h in range(heads)), dim, 10000.0)
+    att = DifferentialAttentionConfig(heads, kv_heads, dim // 2, dim, (dim // 2) ** -0.5, 0.5,
+                                      window, 4)
+    layers, first_l = [], -1
+    for j in range(0, len(pattern), 2):
+        mx_, f = pattern[j], pattern[j + 1]
+        kw = {}
+        if f == "d":
+            kw = {"ff": ff, "limit": 7.0}
+        elif f == "e":
+            kw = {"moe": ScaledMoeConfig(experts, top, expert_ff or max(8, ff // max(1, top)), 1.5,
+                                         shared_ff)}
+        if mx_ == "r":
+            layers.append(TofodraLayerConfig("retention", ret, **kw))
+        elif mx_ == "a":
+            layers.append(TofodraLayerConfig("attention", att, **kw))
+        else:
+            lat = LatentAttentionConfig(heads, dim, rot_dim, dim, kv_rank, 0, rot_dim, 10000.0,
+                                        (dim + rot_dim) ** -0.5, first_l if mx_ == "s" else -1)
+            if mx_ == "l" and first_l < 0:
+                first_l = j // 2
+            layers.append(TofodraLayerConfig("latent_attention", lat, **kw))
+    return TofodraConfig(name=name, vocab_size=vocab, hidden_size=width, layers=tuple(layers),
+                         embed_scale=8.0)
+
+
+HYBRID_PRESETS.update({
+    "tofodra-tiny": tofodra_preset("tofodra-tiny", 512, 128, 192, "rdaeldsere", 4, 2, 32, 48, 24, 6,
+                                   2, 48, 16, 40),
+    # the "small" Llama preset's geometry (width 1024, 8 q / 2 kv heads of 128, FFN 2816, 4 layers)
+    "tofodra-small": tofodra_preset("tofodra-small", 32768, 1024, 2816, "rdaeldrd", 8, 2, 128, 192,
+                                    1024, 8, 2, 1408),
+    # Llama-3.2-3B / Llama-3.1-8B layer geometry, one layer per mixer
+    "tofodra-3b-slice": tofodra_preset("tofodra-3b-slice", 16384, 3072, 8192, "rdaeld", 24, 8, 128,
+                                       192, 1024, 8, 2, 4096),
+    "tofodra-8b-slice": tofodra_preset("tofodra-8b-slice", 16384, 4096, 14336, "rdaeld", 32, 8, 128,
+                                       192, 1024, 8, 2, 7168),
+})
+ARCHITECTURES["Tofodra"] = TofodraConfig.from_dict
 
 
 def resolve_model(model: str) -> tuple[ModelConfig, str | None]:

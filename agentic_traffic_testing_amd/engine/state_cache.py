@@ -26,13 +26,15 @@ class LayerCacheSpec:
     state_vdim: int = 0
     conv_channels: int = 0     # > 0: tails [slots, conv_taps - 1, conv_channels]
     conv_taps: int = 0
+    v_heads: int = 0           # > 0: V pages hold this many heads (fewer than kv_heads: shared values)
     kv_from: int = -1          # >= 0: no pages of its own, the layer reads that layer's K / V
     shift_channels: int = 0    # > 0: fp32 [slots, shift_channels], the previous token's mixer input
 
     def page_bytes(self, block_size: int, itemsize: int) -> int:
         if self.kv_from >= 0:
             return 0
-        return self.kv_heads * block_size * (self.kdim + self.vdim) * itemsize
+        return block_size * (self.kv_heads * self.kdim
+                             + (self.v_heads or self.kv_heads) * self.vdim) * itemsize
 
     def slot_bytes(self, itemsize: int) -> int:
         return (self.state_heads * self.state_dim * self.state_vdim * 4
@@ -69,8 +71,8 @@ class HybridCache:
             elif sp.kv_heads:
                 lc.k = torch.zeros(num_blocks, sp.kv_heads, block_size, sp.kdim, dtype=dtype,
                                    device=device)
-                lc.v = torch.zeros(num_blocks, sp.kv_heads, sp.vdim, block_size, dtype=dtype,
-                                   device=device)
+                lc.v = torch.zeros(num_blocks, sp.v_heads or sp.kv_heads, sp.vdim, block_size,
+                                   dtype=dtype, device=device)
             if sp.state_heads:
                 lc.state = torch.zeros(num_slots, sp.state_heads, sp.state_dim, sp.state_vdim,
                                        dtype=torch.float32, device=device)

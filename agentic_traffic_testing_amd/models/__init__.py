@@ -27,7 +27,11 @@ def model_class(family: str):
         from .kolotar import KolotarModel
 
         return KolotarModel
+    if family == "tofodra":
+        from .tofodra import TofodraModel
+
+        return TofodraModel
     raise ValueError(f"no model registered for family {family!r}")
 
 
-FAMILIES = ("llama", "ledazen", "soselix", "semezen", "lovapel", "kolotar")
+FAMILIES = ("llama", "ledazen", "soselix", "semezen", "lovapel", "kolotar", "tofodra")

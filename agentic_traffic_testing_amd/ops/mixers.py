@@ -10,7 +10,9 @@ correction and group-limited choice; identity experts), the sandwich-norm layer 
 norm or RMS norm of a branch added to the fp32 residual, then the next norm), the post-norm
 boundary (the residual itself normed after a weighted sum), q / k norms over a whole projection,
 values normed per head and mixed with an earlier layer's, a position-dependent query temperature,
-unnormalised sigmoid attention with head mixing, and scaled, soft-capped logits.
+unnormalised sigmoid attention with head mixing, scaled, soft-capped logits, retention (linear
+attention with a fixed decay per head), and differential attention (two softmax maps over the same
+values) inside windows that keep a sequence's first tokens.
 
 Same device-strict dispatch as ``ops``: GPU tensors run the HIP kernels of
 ``ops/csrc/mixers`` (library ``_atta_mixers.so``, operators ``torch.ops.atta_mix.*``; built on
@@ -204,7 +206,7 @@ def mfma_attention_ok(q, k_cache, v_cache) -> bool:
 
 def sink_attention(q, k_cache, v_cache, block_tables, seq_kvlen, seq_qstart, tile_seq, tile_qoff,
                    scale, sink=True, num_decode=0, max_decode_kv=0, sink_values=None, window=0,
-                   gate=None):
+                   gate=None, keep_first=0, out_dtype=None):
     """Causal attention of every portion's rows over its sequence's pages
     (k_cache [nb, G, BS, d], v_cache [nb, G, dv, BS]).  Sequences [0, num_decode) have one
     query row each and go through the partitioned decode kernel (``max_decode_kv``: their
@@ -212,26 +214,66 @@ def sink_attention(q, k_cache, v_cache, block_tables, seq_kvlen, seq_qstart, til
     ATTN_TILE_TOKENS query rows of every other portion (sequence index, row offset in it).
     ``sink_values``: fp32 [H], the sink's (unscaled) score per query head instead of 0.
     ``window`` > 0: a row at position i sees keys j with 0 <= i - j < window (decode then runs
-    only the partitions that overlap the window).
-    ``gate`` [T, H] (row-strided): head h's output of row t is multiplied by sigmoid(gate[t, h])."""
-    window = int(window)
+    only the partitions that overlap the window); with ``keep_first`` it also sees the keys
+    j < keep_first, however far back.
+    ``gate`` [T, H] (row-strided): head h's output of row t is multiplied by sigmoid(gate[t, h]).
+    q [T, H, d] may be row-strided.  A V cache with fewer heads than the K cache serves an equal
+    run of neighbouring K heads with each of its heads.  ``out_dtype`` float32: results are stored
+    unrounded whatever q's dtype."""
+    window, keep_first = int(window), int(keep_first) if window > 0 else 0
     if not q.is_cuda:
         return mref.sink_attention(q, k_cache, v_cache, block_tables, seq_kvlen, seq_qstart,
-                                   scale, sink, sink_values, window, gate)
-    out = torch.empty(q.shape[0], q.shape[1], v_cache.shape[2], dtype=q.dtype, device=q.device)
+                                   scale, sink, sink_values, window, gate, keep_first, out_dtype)
+    out = torch.empty(q.shape[0], q.shape[1], v_cache.shape[2], dtype=out_dtype or q.dtype,
+                      device=q.device)
     part = None
     if num_decode > 0:
         parts = max(1, -(-int(max_decode_kv) // DECODE_PART_TOKENS))
         if window > 0:   # the window touches at most this many partitions
-            parts = min(parts, -(-window // DECODE_PART_TOKENS) + 1)
+            parts = min(parts, -(-window // DECODE_PART_TOKENS) + 1
+                        + -(-keep_first // DECODE_PART_TOKENS))
         part = torch.empty(num_decode, q.shape[1], parts, v_cache.shape[2] + 2,
                            dtype=torch.float32, device=q.device)
     if tile_seq.shape[0] > 0 or num_decode > 0:
         _native().sink_attention(out, q, k_cache, v_cache, block_tables, seq_kvlen, seq_qstart,
                                  tile_seq, tile_qoff, scale, sink, num_decode,
                                  max(1, int(max_decode_kv)), part,
-                                 mfma_attention_ok(q, k_cache, v_cache), sink_values, window, gate)
+                                 mfma_attention_ok(q, k_cache, v_cache), sink_values, window, gate,
+                                 keep_first)
     return out
+
+
+def kv_cache_write(kx, vx, slot_mapping, k_cache, v_cache):
+    """Rows kx [T, G * d] and vx [T, GV * dv] (row-strided) as they are into the pages k_cache
+    [nb, G, BS, d] and the channel-major pages v_cache [nb, GV, dv, BS]."""
+    if not kx.is_cuda:
+        return mref.kv_cache_write(kx, vx, slot_mapping, k_cache, v_cache)
+    _native().kv_cache_write(kx, vx, slot_mapping, k_cache, v_cache)
+
+
+def diff_combine(a, gate, lam, diff, eps, kv_heads, dtype=torch.bfloat16):
+    """Joins the two maps of differential attention.  a fp32 [T, 2 H, dv], heads in the order
+    (KV head, map, head of the group); per head o = a1 - lam a2, divided by its root mean square
+    over dv, times (1 - diff) and, with a gate [T, H * dv] (row-strided), sigmoid(gate) ->
+    [T, H * dv] in ``dtype``."""
+    if not a.is_cuda:
+        return mref.diff_combine(a, gate, float(lam), float(diff), eps, kv_heads, dtype)
+    out = torch.empty(a.shape[0], a.shape[1] // 2 * a.shape[2], dtype=dtype, device=a.device)
+    _native().diff_combine(out, a, gate, float(lam), float(diff), eps, kv_heads)
+    return out
+
+
+def differential_attention(q, k_cache, v_cache, block_tables, seq_kvlen, seq_qstart, tile_seq,
+                           tile_qoff, scale, lam, diff, eps, gate=None, num_decode=0,
+                           max_decode_kv=0, window=0, keep_first=0):
+    """Two softmax maps over the same values: q [T, 2 H, d] (row-strided) and k_cache
+    [nb, 2 G, BS, d] hold the heads in the order (KV head, map, head of the group), v_cache
+    [nb, G, dv, BS] is shared by the maps; returns ``diff_combine`` of the two
+    ([T, H * dv], q's dtype).  Batch layout, window and ``keep_first`` as in ``sink_attention``."""
+    a = sink_attention(q, k_cache, v_cache, block_tables, seq_kvlen, seq_qstart, tile_seq, tile_qoff,
+                       scale, False, num_decode, max_decode_kv, window=window,
+                       keep_first=keep_first, out_dtype=torch.float32)
+    return diff_combine(a, gate, lam, diff, eps, v_cache.shape[1], q.dtype)
 
 
 def sigmoid_attention(q, k_cache, v_cache, block_tables, seq_kvlen, seq_qstart, tile_seq,
@@ -289,6 +331,8 @@ def gated_delta_rule(qkv, beta_logit, decay_logit, a_log, dt_bias, state, positi
 
 
 def gated_rms_norm(o, gate, w, eps, act="silu", dtype=torch.bfloat16):
+    """fp32 o [T, H, dv] divided by its root mean square per head, times w [dv] (None: no weight)
+    and act(gate [T, H * dv], row-strided) -> [T, H * dv]."""
     if not o.is_cuda:
         return mref.gated_rms_norm(o, gate, w, eps, act, dtype)
     T, H, dv = o.shape
@@ -365,7 +409,7 @@ def group_rms_norm(y, gate, w, n_groups, eps, dtype=torch.bfloat16):
 
 def head_gate(o, gate):
     """o [H, T, dv] (head-major) times sigmoid(gate) -> [T, H * dv]; gate [T, H] (one number per
-    head) or [T, H * dv] (one per channel)."""
+    head), [T, H * dv] (one per channel) or None (the move alone)."""
     if not o.is_cuda:
         return mref.head_gate(o, gate)
     H, T, dv = o.shape
@@ -426,6 +470,33 @@ def state_space_scan(x, B, C, dt, dt_bias, a_log, skip, state, positions, seq_qs
 
 
 
+RETENTION_CHUNK = 64      # tokens per chunk of the matrix-core prefill kernel
+
+
+def retention_powers(decay, device) -> torch.Tensor:
+    """fp32 [heads, RETENTION_CHUNK + 1] of decay^n (computed in float64, rounded once): the weights
+    inside a chunk and the decay over it; column 1 is the decay itself."""
+    d = torch.tensor([float(x) for x in decay], dtype=torch.float64)
+    n = torch.arange(RETENTION_CHUNK + 1, dtype=torch.float64)
+    return torch.pow(d[:, None], n[None, :]).to(torch.float32).to(device)
+
+
+def retention(q, k, v, powers, cos_sin, state, positions, seq_qstart, seq_slot, heads, dim, vdim,
+              num_decode=0):
+    """Linear attention with a fixed decay per head: S = decay S + k v^T, o = S^T q, with
+    rotate-half positions (table ``cos_sin`` [T, 2 n], n <= dim / 2) on q and k and k times
+    dim^-0.5, all in fp32.  q, k [T, heads * dim], v [T, heads * vdim] (row-strided); ``powers``:
+    ``retention_powers``; state fp32 [slots, heads, dim, vdim] advanced in place; returns fp32
+    [T, heads, vdim].  Sequences [0, num_decode) have one row each."""
+    if not v.is_cuda:
+        return mref.retention(q, k, v, powers[:, 1], cos_sin, state, positions, seq_qstart, seq_slot,
+                              heads, dim, vdim)
+    out = torch.empty(v.shape[0], heads, vdim, dtype=torch.float32, device=v.device)
+    _native().retention(out, state, q, k, v, powers, cos_sin, positions, seq_qstart, seq_slot, heads,
+                        dim, vdim, int(num_decode))
+    return out
+
+
 def hyper_norm(xs, w_in, w, eps, dtype=torch.bfloat16):
     """xs fp32 [T, s, W] (the residual streams): RMS norm with weight ``w`` of
     u = sum_s w_in[s] xs[:, s] -> [T, W] of ``dtype``.  w_in fp32 [s]."""
@@ -468,6 +539,16 @@ def gate_mul(a, gate, act="sigmoid"):
         return mref.gate_mul(a, gate, code)
     out = torch.empty(a.shape, dtype=a.dtype, device=a.device)
     _native().gate_mul(out, a, gate, code)
+    return out
+
+
+def clamped_gate_mul(up, gate, limit, alpha=1.702):
+    """Clamped GLU of two products [T, N] (row-strided slices of a fused projection):
+    g sigmoid(alpha g) (u + 1) with g = min(gate, limit), u = clamp(up, -limit, limit)."""
+    if not up.is_cuda:
+        return mref.clamped_gate_mul(up, gate, float(limit), float(alpha))
+    out = torch.empty(up.shape, dtype=up.dtype, device=up.device)
+    _native().clamped_glu(out, gate, up, None, float(limit), float(alpha))
     return out
 
 
@@ -515,7 +596,8 @@ def clamped_glu(gu, wts, limit, alpha=1.702):
     if not gu.is_cuda:
         return mref.clamped_glu(gu, wts, limit, alpha)
     out = torch.empty(gu.shape[0], gu.shape[1] // 2, dtype=gu.dtype, device=gu.device)
-    _native().clamped_glu(out, gu, wts, float(limit), float(alpha))
+    ff = out.shape[1]
+    _native().clamped_glu(out, gu[:, :ff], gu[:, ff:], wts, float(limit), float(alpha))
     return out
 
 
@@ -556,24 +638,26 @@ def _moe_experts_library(h, idx, wts, w_gu, w_down, limit, alpha, silu_glu=False
     return _pair_sum(y, T, k)
 
 
-def moe_route(logits, top, score="sigmoid", correction=None, groups=1, keep=1, renorm=False):
+def moe_route(logits, top, score="sigmoid", correction=None, groups=1, keep=1, renorm=False,
+              scale=1.0):
     """fp32 router logits [T, E] -> (expert index int32 [T, top], score fp32 [T, top]) of every
     row's ``top`` largest scores (ties: lowest index).  ``score``: "sigmoid", "softmax" over
     the row, or "logit" (the logits choose, the weights are their softmax over the chosen ones).
     ``correction`` fp32 [E] is added to the scores for the choice only (the returned weights are
     the plain scores).  ``groups`` > 1: the experts form that many equal runs of
     neighbours, a group's score is its largest choice score, and only experts of the ``keep``
-    best groups can be chosen.  ``renorm``: the chosen scores are divided by their sum + 1e-20."""
+    best groups can be chosen.  ``renorm``: the chosen scores are divided by their sum + 1e-20;
+    ``scale`` multiplies the weights."""
     E = logits.shape[1]
     code = _SCORE_CODES[score]
     if groups < 1 or E % groups or not 1 <= keep <= groups or top > keep * (E // groups):
         raise ValueError("moe_route: groups must split the experts evenly and hold `top` of them")
     if not logits.is_cuda:
-        return mref.moe_route(logits, top, score, correction, groups, keep, renorm)
+        return mref.moe_route(logits, top, score, correction, groups, keep, renorm, float(scale))
     T = logits.shape[0]
     idx = torch.empty(T, top, dtype=torch.int32, device=logits.device)
     wts = torch.empty(T, top, dtype=torch.float32, device=logits.device)
-    _native().moe_route(idx, wts, logits, code, correction, groups, keep, renorm)
+    _native().moe_route(idx, wts, logits, code, correction, groups, keep, renorm, float(scale))
     return idx, wts
 
 
@@ -624,17 +708,18 @@ def moe_experts(h, idx, wts, w_gu, w_down, limit=0.0, alpha=1.702, glu="clamped"
     return _pair_sum(y, T, k * split, h.dtype)
 
 
-def norm_add_norm(x, y, w_post, w_next, eps, kind="layer", dtype=torch.bfloat16):
+def norm_add_norm(x, y, w_post, w_next, eps, kind="layer", dtype=torch.bfloat16, post_scale=None):
     """Layer boundary of a sandwich-norm residual in one pass: x (fp32 [T, W], in place) +=
-    norm(y) * w_post (y None: nothing is added), then returns norm(x) * w_next in ``dtype``
+    norm(y) * w_post (y None: nothing is added; ``post_scale`` [W]: a per-channel scale of the
+    branch, multiplied on top), then returns norm(x) * w_next in ``dtype``
     (None when ``w_next`` is None).  ``kind`` "layer": (v - mean) / sqrt(var + eps) with var the
     mean squared deviation; "rms": v / sqrt(mean(v^2) + eps).  Sums and statistics in fp32."""
     if kind not in ("layer", "rms"):
         raise ValueError(kind)
     if not x.is_cuda:
-        return mref.norm_add_norm(x, y, w_post, w_next, eps, kind == "layer", dtype)
+        return mref.norm_add_norm(x, y, w_post, w_next, eps, kind == "layer", dtype, post_scale)
     h = torch.empty(x.shape, dtype=dtype, device=x.device) if w_next is not None else None
-    _native().norm_add_norm(h, x, y, w_post, w_next, eps, kind == "layer")
+    _native().norm_add_norm(h, x, y, w_post, w_next, post_scale, eps, kind == "layer")
     return h
 
 

@@ -119,15 +119,17 @@ def qk_norm_rope_cache(qx, kx, vx, q_norm, k_norm, eps, positions, slot_mapping,
 
 
 def sink_attention(q, k_cache, v_cache, block_tables, seq_kvlen, seq_qstart, scale, sink,
-                   sink_values=None, window=0, gate=None):
+                   sink_values=None, window=0, gate=None, keep_first=0, out_dtype=None):
     """Causal paged attention of every portion's rows over its sequence's cached keys; fp32
     scores and weights; ``sink`` adds exp(s - max) to each denominator, s = 0 or the head's
     entry of ``sink_values`` [H]; ``window`` > 0: a row at position i sees keys j with
-    0 <= i - j < window; ``gate`` [T, H]: outputs times sigmoid(gate).  q [T, H, d] ->
-    [T, H, dv]."""
+    0 <= i - j < window, and those with j < ``keep_first``; ``gate`` [T, H]: outputs times
+    sigmoid(gate).  A V cache with fewer heads than the K cache serves an equal run of neighbouring
+    K heads with each of its heads.  q [T, H, d] -> [T, H, dv] (of ``out_dtype``)."""
     T, H, _ = q.shape
     G, bs, dv = k_cache.shape[1], k_cache.shape[2], v_cache.shape[2]
-    out = torch.zeros(T, H, dv, dtype=q.dtype, device=q.device)
+    GV = v_cache.shape[1]
+    out = torch.zeros(T, H, dv, dtype=out_dtype or q.dtype, device=q.device)
     qs = seq_qstart.tolist()
     for s, kvlen in enumerate(seq_kvlen.tolist()):
         a, b = qs[s], qs[s + 1]
@@ -136,16 +138,16 @@ def sink_attention(q, k_cache, v_cache, block_tables, seq_kvlen, seq_qstart, sca
         nblk = (kvlen + bs - 1) // bs
         pages = block_tables[s, :nblk].long()
         k = k_cache[pages].permute(1, 0, 2, 3).reshape(G, nblk * bs, -1)[:, :kvlen].float()
-        v = v_cache[pages].permute(1, 0, 3, 2).reshape(G, nblk * bs, dv)[:, :kvlen].float()
+        v = v_cache[pages].permute(1, 0, 3, 2).reshape(GV, nblk * bs, dv)[:, :kvlen].float()
         k = k.repeat_interleave(H // G, 0)
-        v = v.repeat_interleave(H // G, 0)
+        v = v.repeat_interleave(H // GV, 0)
         n = b - a
         sc = torch.einsum("qhd,hkd->hqk", q[a:b].float(), k) * scale
         qpos = torch.arange(kvlen - n, kvlen, device=q.device)
         kpos = torch.arange(kvlen, device=q.device)
         mask = kpos[None, :] > qpos[:, None]
         if window > 0:
-            mask = mask | (kpos[None, :] <= qpos[:, None] - window)
+            mask = mask | ((kpos[None, :] <= qpos[:, None] - window) & (kpos[None, :] >= keep_first))
         sc = sc.masked_fill(mask[None], float("-inf"))
         m = sc.amax(-1, keepdim=True)
         if sink:
@@ -159,7 +161,7 @@ def sink_attention(q, k_cache, v_cache, block_tables, seq_kvlen, seq_qstart, sca
         o = torch.einsum("hqk,hkd->qhd", e / den, v)
         if gate is not None:
             o = o * torch.sigmoid(gate[a:b].float())[:, :, None]
-        out[a:b] = o.to(q.dtype)
+        out[a:b] = o.to(out.dtype)
     return out
 
 
@@ -259,11 +261,14 @@ def gated_delta_rule(qkv, beta_logit, decay_logit, a_log, dt_bias, state, positi
 
 
 def gated_rms_norm(o, gate, w, eps, act, dtype):
-    """o fp32 [T, H, dv] / rms over dv * w [dv] * act(gate [T, H * dv]) -> [T, H * dv]."""
+    """o fp32 [T, H, dv] / rms over dv * w [dv] (None: no weight) * act(gate [T, H * dv]) ->
+    [T, H * dv]."""
     T, H, dv = o.shape
     g = gate.float().view(T, H, dv)
     g = torch.sigmoid(g) if act == "sigmoid" else g * torch.sigmoid(g)
-    y = o * torch.rsqrt(o.pow(2).mean(-1, keepdim=True) + eps) * w.float() * g
+    y = o * torch.rsqrt(o.pow(2).mean(-1, keepdim=True) + eps) * g
+    if w is not None:
+        y = y * w.float()
     return y.to(dtype).view(T, H * dv)
 
 
@@ -316,6 +321,8 @@ def group_rms_norm(y, gate, w, n_groups, eps, dtype):
 
 def head_gate(o, gate):
     H, T, dv = o.shape
+    if gate is None:
+        return o.permute(1, 0, 2).reshape(T, H * dv)
     g = torch.sigmoid(gate.float())                       # [T, H] or [T, H * dv]
     g = g[:, :, None] if g.shape[1] == H else g.reshape(T, H, dv)
     return (o.float().permute(1, 0, 2) * g).to(o.dtype).reshape(T, H * dv)
@@ -465,12 +472,14 @@ def gelu(x, tanh_form=False):
     return F.gelu(x.float(), approximate="tanh" if tanh_form else "none").to(x.dtype)
 
 
-def moe_route(logits, top, score="sigmoid", correction=None, groups=1, keep=1, renorm=False):
+def moe_route(logits, top, score="sigmoid", correction=None, groups=1, keep=1, renorm=False,
+              scale=1.0):
     """Scores (sigmoid, softmax over the row, or the logits themselves) of fp32 router logits [T, E]; the ``top`` largest
     per row (ties: lowest index) -> (int32 [T, top], fp32 [T, top]).  ``correction`` [E] is added
     to the scores for the choice only; with ``groups`` > 1 only experts of the ``keep`` groups (equal
     runs of neighbours) with the largest best choice score can be chosen; ``renorm``: the chosen
-    scores are divided by their sum + 1e-20; "logit" scores give the softmax over the chosen."""
+    scores are divided by their sum + 1e-20; "logit" scores give the softmax over the chosen;
+    ``scale`` multiplies the weights."""
     z = logits.float()
     s = {"softmax": lambda: torch.softmax(z, 1), "sigmoid": lambda: torch.sigmoid(z),
          "logit": lambda: z}[score]()
@@ -488,7 +497,7 @@ def moe_route(logits, top, score="sigmoid", correction=None, groups=1, keep=1, r
         w = torch.softmax(w, 1)
     elif renorm:
         w = w / (w.sum(1, keepdim=True) + 1e-20)
-    return order.to(torch.int32), w
+    return order.to(torch.int32), w * scale if scale != 1.0 else w
 
 
 def moe_experts(h, idx, wts, w_gu, w_down, limit, alpha, silu_glu=False, addend=None):
@@ -535,8 +544,9 @@ def moe_experts_silu(h, idx, wts, w_gu, w_down, addend=None):
     return out.to(h.dtype)
 
 
-def norm_add_norm(x, y, w_post, w_next, eps, layer, dtype):
-    """x (fp32 [T, W], in place) += norm(y) * w_post (nothing when y is None); returns
+def norm_add_norm(x, y, w_post, w_next, eps, layer, dtype, post_scale=None):
+    """x (fp32 [T, W], in place) += norm(y) * w_post (nothing when y is None; times ``post_scale``
+    [W] when given); returns
     norm(x) * w_next in ``dtype`` (None when w_next is None).  norm: the layer norm
     (x - mean) / sqrt(var + eps) when ``layer``, else x / sqrt(mean(x^2) + eps); all in fp32."""
     def nrm(v, w):
@@ -546,7 +556,7 @@ def norm_add_norm(x, y, w_post, w_next, eps, layer, dtype):
         return v * torch.rsqrt(v.pow(2).mean(-1, keepdim=True) + eps) * w.float()
 
     if y is not None:
-        x += nrm(y, w_post)
+        x += nrm(y, w_post) if post_scale is None else nrm(y, w_post) * post_scale.float()
     return nrm(x, w_next).to(dtype) if w_next is not None else None
 
 
@@ -574,3 +584,59 @@ def clamped_glu(gu, wts, limit, alpha):
     g = (gu[:, :ff].float() * w).clamp(max=limit)
     u = (gu[:, ff:].float() * w).clamp(-limit, limit)
     return (g * torch.sigmoid(alpha * g) * (u + 1.0)).to(gu.dtype)
+
+
+def clamped_gate_mul(up, gate, limit, alpha=1.702):
+    """Clamped GLU of two products [T, N]: g sigmoid(alpha g) (u + 1), g = min(gate, limit),
+    u = clamp(up, -limit, limit)."""
+    g = gate.float().clamp(max=limit)
+    u = up.float().clamp(-limit, limit)
+    return (g * torch.sigmoid(alpha * g) * (u + 1.0)).to(up.dtype)
+
+
+# ---- retention, differential attention ---------------------------------------------------------
+
+def kv_cache_write(kx, vx, slot_mapping, k_cache, v_cache):
+    """Rows kx [T, G * d] and vx [T, GV * dv] as they are into the paged caches k_cache
+    [nb, G, BS, d], v_cache [nb, GV, dv, BS] (rows with slot -1 excepted)."""
+    G, bs, d = k_cache.shape[1:]
+    GV, dv = v_cache.shape[1:3]
+    sm = slot_mapping.long()[:kx.shape[0]]
+    ok = sm >= 0
+    if bool(ok.any()):
+        s = sm[ok]
+        k_cache[s // bs, :, s % bs, :] = kx[ok].reshape(-1, G, d)
+        v_cache[s // bs, :, :, s % bs] = vx[ok].reshape(-1, GV, dv)
+
+
+def diff_combine(a, gate, lam, diff, eps, kv_heads, dtype):
+    """a fp32 [T, 2 H, dv], the heads in the order (KV head, map, head of the group): per head
+    o = a1 - lam a2, divided by its root mean square, times (1 - diff) and sigmoid(gate [T, H dv])
+    -> [T, H * dv]."""
+    T, H2, dv = a.shape
+    a = a.float().view(T, kv_heads, 2, H2 // (2 * kv_heads), dv)
+    o = a[:, :, 0] - lam * a[:, :, 1]
+    o = o * torch.rsqrt(o.pow(2).mean(-1, keepdim=True) + eps) * (1.0 - diff)
+    o = o.reshape(T, H2 // 2 * dv)
+    return (o * torch.sigmoid(gate.float()) if gate is not None else o).to(dtype)
+
+
+def retention(q, k, v, decay, cos_sin, state, positions, seq_qstart, seq_slot, heads, dim, vdim):
+    """Per head S = decay S + k v^T, o = S^T q with rotate-half positions on q and k and k times
+    dim^-0.5.  q, k [T, heads * dim], v [T, heads * vdim] (row-strided); decay fp32 [heads]; state
+    fp32 [slots, heads, dim, vdim] advanced in place; returns fp32 [T, heads, vdim]."""
+    T = v.shape[0]
+    qq = rotate_half(q.float().reshape(T, heads, dim), cos_sin)
+    kk = rotate_half(k.float().reshape(T, heads, dim), cos_sin) * dim ** -0.5
+    vv = v.float().reshape(T, heads, vdim)
+    out = torch.zeros(T, heads, vdim, dtype=torch.float32, device=v.device)
+    g = decay.float()[:, None, None]
+    for s, slot, b0, b1 in _portions(seq_qstart, seq_slot):
+        S = state[slot].clone()
+        if int(positions[b0]) == 0:
+            S.zero_()
+        for t in range(b0, b1):
+            S = g * S + kk[t][:, :, None] * vv[t][:, None, :]
+            out[t] = torch.einsum("hdv,hd->hv", S, qq[t])
+        state[slot] = S
+    return out
