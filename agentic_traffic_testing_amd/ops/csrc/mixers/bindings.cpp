@@ -134,18 +134,19 @@ void add_norm(at::Tensor h, at::Tensor x, const at::Tensor& a, double sa,
 }
 
 void gated_rms_norm(at::Tensor out, const at::Tensor& o, const at::Tensor& gate,
-                    const at::Tensor& w, double eps, int64_t act) {
+                    const c10::optional<at::Tensor>& w, double eps, int64_t act) {
   f32c(o, "o");
   TORCH_CHECK(o.dim() == 3, "gated_rms_norm: o [T, H, dv]");
   const int64_t T = o.size(0), H = o.size(1), dv = o.size(2);
   rows2d(gate, out, "gate");
   TORCH_CHECK(gate.size(0) == T && gate.size(1) == H * dv && out.is_contiguous() &&
-                  out.numel() == o.numel() && w.is_contiguous() && w.numel() == dv &&
-                  w.scalar_type() == out.scalar_type(),
+                  out.numel() == o.numel() &&
+                  (!w || (w->is_cuda() && w->is_contiguous() && w->numel() == dv &&
+                          w->scalar_type() == out.scalar_type())),
               "gated_rms_norm: shapes");
   const at::DeviceGuard g(o.device());
   rc_ok(mixk_gated_rms_norm(out.data_ptr(), o.data_ptr<float>(), gate.data_ptr(), gate.stride(0),
-                            w.data_ptr(), T, H, dv, static_cast<float>(eps), act, code(out),
+                            w ? w->data_ptr() : nullptr, T, H, dv, static_cast<float>(eps), act, code(out),
                             cur_stream()),
         "gated_rms_norm");
 }
@@ -233,6 +234,8 @@ void rotary_table(at::Tensor out, const at::Tensor& positions, const at::Tensor&
         "rotary_table");
 }
 
+// `pair` (differential attention): {lambda, factor after the norm, eps}; H counts both maps, out is
+// [T, H / 2, dv] of q's dtype and gate [T, H / 2 * dv].
 void sink_attention(at::Tensor out, const at::Tensor& q, const at::Tensor& k_cache,
                     const at::Tensor& v_cache, const at::Tensor& block_tables,
                     const at::Tensor& seq_kvlen, const at::Tensor& seq_qstart,
@@ -240,27 +243,33 @@ void sink_attention(at::Tensor out, const at::Tensor& q, const at::Tensor& k_cac
                     bool sink, int64_t num_decode, int64_t max_decode_kv,
                     const c10::optional<at::Tensor>& part, bool use_mfma,
                     const c10::optional<at::Tensor>& sink_val, int64_t window,
-                    const c10::optional<at::Tensor>& gate) {
-  TORCH_CHECK(q.is_cuda() && q.dim() == 3 && q.is_contiguous() && out.dim() == 3 &&
-                  out.is_contiguous() && k_cache.dim() == 4 && v_cache.dim() == 4 &&
-                  k_cache.is_contiguous() && v_cache.is_contiguous(),
-              "sink_attention: q [T, H, d], out [T, H, dv], K [nb, G, BS, d], V [nb, G, dv, BS]");
+                    const c10::optional<at::Tensor>& gate, int64_t keep,
+                    const c10::optional<at::ArrayRef<double>>& pair) {
+  TORCH_CHECK(q.is_cuda() && q.dim() == 3 && q.stride(2) == 1 && q.stride(1) == q.size(2) &&
+                  out.is_cuda() && out.dim() == 3 && out.is_contiguous() && k_cache.dim() == 4 &&
+                  v_cache.dim() == 4 && k_cache.is_contiguous() && v_cache.is_contiguous(),
+              "sink_attention: q [T, H, d], out [T, H, dv], K [nb, G, BS, d], V [nb, GV, dv, BS]");
   const int64_t H = q.size(1), dim = q.size(2), G = k_cache.size(1), BS = k_cache.size(2);
-  const int64_t vdim = v_cache.size(2), S = seq_kvlen.numel();
+  const int64_t vdim = v_cache.size(2), S = seq_kvlen.numel(), GV = v_cache.size(1);
   i32(block_tables, "block_tables");
   i32(seq_kvlen, "seq_kvlen");
   i32(seq_qstart, "seq_qstart");
   i32(tile_seq, "tile_seq");
   i32(tile_qoff, "tile_qoff");
+  const bool out_f32 = out.scalar_type() == at::kFloat;
   TORCH_CHECK(block_tables.dim() == 2 && block_tables.size(0) >= S &&
                   seq_qstart.numel() == S + 1 && tile_seq.numel() == tile_qoff.numel() &&
-                  out.size(0) == q.size(0) && out.size(1) == H && out.size(2) == vdim &&
-                  k_cache.size(3) == dim && v_cache.size(1) == G && v_cache.size(3) == BS &&
-                  v_cache.size(0) == k_cache.size(0) && H % G == 0 &&
-                  out.scalar_type() == q.scalar_type() &&
-                  k_cache.scalar_type() == q.scalar_type() &&
+                  out.size(0) == q.size(0) && out.size(1) == (pair ? H / 2 : H) &&
+                  out.size(2) == vdim && k_cache.size(3) == dim && GV > 0 && G % GV == 0 &&
+                  v_cache.size(3) == BS && v_cache.size(0) == k_cache.size(0) && H % G == 0 &&
+                  (out.scalar_type() == q.scalar_type() || (out_f32 && !pair)) &&
+                  k_cache.scalar_type() == q.scalar_type() && keep >= 0 &&
                   v_cache.scalar_type() == q.scalar_type() && num_decode >= 0 && num_decode <= S,
               "sink_attention: shapes");
+  if (pair)
+    TORCH_CHECK(pair->size() == 3 && use_mfma && !sink && G == 2 * GV,
+                "sink_attention: the pair form is the matrix-core kernel's, without a sink, two K "
+                "heads per V head");
   float* part_ptr = nullptr;
   int64_t max_parts = 0;
   if (num_decode > 0) {
@@ -269,16 +278,18 @@ void sink_attention(at::Tensor out, const at::Tensor& q, const at::Tensor& k_cac
     TORCH_CHECK(part->dim() == 4 && part->size(0) >= num_decode && part->size(1) == H &&
                     part->size(3) == vdim + 2 && max_decode_kv >= 1 && window >= 0 &&
                     (part->size(2) * 128 >= max_decode_kv ||
-                     (window > 0 && part->size(2) >= (window + 127) / 128 + 1)),
+                     (window > 0 &&
+                      part->size(2) >= (window + 127) / 128 + 1 + (keep + 127) / 128)),
                 "sink_attention: partials [num_decode, H, parts, vdim + 2]");
     part_ptr = part->data_ptr<float>();
     max_parts = part->size(2);
   }
   if (use_mfma)
     TORCH_CHECK(q.scalar_type() == at::kBFloat16 && dim % 16 == 0 && vdim % 32 == 0 &&
-                    dim <= 256 && vdim <= 256 && BS >= 8 && (BS & (BS - 1)) == 0,
+                    dim <= 256 && vdim <= 256 && BS >= 8 && (BS & (BS - 1)) == 0 &&
+                    q.stride(0) % 8 == 0 && reinterpret_cast<uintptr_t>(q.data_ptr()) % 16 == 0,
                 "sink_attention: matrix-core kernel needs bf16, dim % 16, vdim % 32, <= 256, "
-                "pages of a power of two >= 8 tokens");
+                "16-byte aligned query rows, pages of a power of two >= 8 tokens");
   const float* sink_ptr = nullptr;
   if (sink_val) {
     f32c(*sink_val, "sink_val");
@@ -287,7 +298,10 @@ void sink_attention(at::Tensor out, const at::Tensor& q, const at::Tensor& k_cac
   }
   if (gate) {
     rows2d(*gate, q, "gate");
-    TORCH_CHECK(gate->size(0) == q.size(0) && gate->size(1) == H, "sink_attention: gate [T, H]");
+    TORCH_CHECK(gate->size(0) == q.size(0) && gate->size(1) == (pair ? H / 2 * vdim : H) &&
+                    (!pair || (gate->stride(0) % 4 == 0 &&
+                               reinterpret_cast<uintptr_t>(gate->data_ptr()) % 8 == 0)),
+                "sink_attention: gate [T, H] (pair form: [T, H / 2 * dv], 8-byte aligned)");
   }
   const at::DeviceGuard g(q.device());
   rc_ok(mixk_sink_attention(out.data_ptr(), q.data_ptr(), k_cache.data_ptr(), v_cache.data_ptr(),
@@ -296,9 +310,90 @@ void sink_attention(at::Tensor out, const at::Tensor& q, const at::Tensor& k_cac
                             tile_seq.data_ptr<int>(), tile_qoff.data_ptr<int>(), tile_seq.numel(),
                             num_decode, max_decode_kv, part_ptr, max_parts, H, G, dim, vdim, BS,
                             static_cast<float>(scale), sink, sink_ptr, static_cast<int>(window),
-                            gate ? gate->data_ptr() : nullptr, gate ? gate->stride(0) : 0,
-                            use_mfma, code(q), cur_stream()),
+                            static_cast<int>(keep), gate ? gate->data_ptr() : nullptr,
+                            gate ? gate->stride(0) : 0, static_cast<int>(G / GV), q.stride(0),
+                            out_f32 && code(q) != 2, pair.has_value(),
+                            pair ? static_cast<float>((*pair)[0]) : 0.f,
+                            pair ? static_cast<float>((*pair)[1]) : 0.f,
+                            pair ? static_cast<float>((*pair)[2]) : 0.f, use_mfma, code(q),
+                            cur_stream()),
         "sink_attention");
+}
+
+// Rows kx [T, GK * d], vx [T, GV * dv] into k_cache [nb, GK, BS, d], v_cache [nb, GV, dv, BS].
+void kv_cache_write(const at::Tensor& kx, const at::Tensor& vx, const at::Tensor& slot_mapping,
+                    at::Tensor k_cache, at::Tensor v_cache) {
+  rows2d(kx, k_cache, "k");
+  rows2d(vx, v_cache, "v");
+  i32(slot_mapping, "slot_mapping");
+  TORCH_CHECK(k_cache.is_cuda() && k_cache.dim() == 4 && v_cache.dim() == 4 &&
+                  k_cache.is_contiguous() && v_cache.is_contiguous() &&
+                  k_cache.scalar_type() == v_cache.scalar_type() &&
+                  k_cache.size(0) == v_cache.size(0) && k_cache.size(2) == v_cache.size(3) &&
+                  kx.size(1) == k_cache.size(1) * k_cache.size(3) &&
+                  vx.size(1) == v_cache.size(1) * v_cache.size(2) && kx.size(0) == vx.size(0) &&
+                  slot_mapping.numel() >= kx.size(0),
+              "kv_cache_write: k [T, G d], v [T, GV dv], caches [nb, G, BS, d], [nb, GV, dv, BS]");
+  const at::DeviceGuard g(kx.device());
+  rc_ok(mixk_kv_cache_write(kx.data_ptr(), kx.stride(0), vx.data_ptr(), vx.stride(0),
+                            slot_mapping.data_ptr<int>(), k_cache.data_ptr(), v_cache.data_ptr(),
+                            kx.size(0), k_cache.size(1), k_cache.size(3), v_cache.size(1),
+                            v_cache.size(2), k_cache.size(2), code(kx), cur_stream()),
+        "kv_cache_write");
+}
+
+// a fp32 [T, 2 HO, dv] in the order (KV head, map, head of the group) -> out [T, HO * dv]
+void diff_combine(at::Tensor out, const at::Tensor& a, const c10::optional<at::Tensor>& gate,
+                  double lam, double diff, double eps, int64_t kv_heads) {
+  f32c(a, "a");
+  TORCH_CHECK(a.dim() == 3 && a.size(1) % 2 == 0 && kv_heads > 0 &&
+                  (a.size(1) / 2) % kv_heads == 0 && out.is_cuda() && out.is_contiguous() &&
+                  out.numel() * 2 == a.numel(),
+              "diff_combine: a [T, 2 H, dv], out [T, H * dv]");
+  const int64_t T = a.size(0), HO = a.size(1) / 2, dv = a.size(2);
+  if (gate) {
+    rows2d(*gate, out, "gate");
+    TORCH_CHECK(gate->size(0) == T && gate->size(1) == HO * dv, "diff_combine: gate [T, H * dv]");
+  }
+  const at::DeviceGuard g(a.device());
+  rc_ok(mixk_diff_combine(out.data_ptr(), a.data_ptr<float>(), gate ? gate->data_ptr() : nullptr,
+                          gate ? gate->stride(0) : 0, T, HO, kv_heads, dv, static_cast<float>(lam),
+                          static_cast<float>(1.0 - diff), static_cast<float>(eps), code(out),
+                          cur_stream()),
+        "diff_combine");
+}
+
+// q, k [T, H dk], v [T, H dv] (row-strided), powers fp32 [H, n] (decay^0 ... decay^(n-1)), cos_sin
+// [rows, 2 n_freq]; sequences [0, num_decode) have one row each.
+void retention(at::Tensor out, at::Tensor state, const at::Tensor& q, const at::Tensor& k,
+               const at::Tensor& v, const at::Tensor& powers, const at::Tensor& cos_sin,
+               const at::Tensor& positions, const at::Tensor& seq_qstart,
+               const at::Tensor& seq_slot, int64_t H, int64_t dk, int64_t dv,
+               int64_t num_decode) {
+  rows2d(v, v, "v");
+  rows2d(q, v, "q");
+  rows2d(k, v, "k");
+  const int64_t T = v.size(0), S = seq_slot.numel();
+  meta(positions, seq_qstart, seq_slot, T);
+  f32c(out, "out");
+  f32c(state, "state");
+  f32c(powers, "powers");
+  f32c(cos_sin, "cos_sin");
+  TORCH_CHECK(H > 0 && dk > 0 && dk <= 256 && dv > 0 && q.size(0) == T && k.size(0) == T &&
+                  q.size(1) == H * dk && k.size(1) == H * dk && v.size(1) == H * dv &&
+                  out.numel() == T * H * dv && state.dim() == 4 && state.size(1) == H &&
+                  state.size(2) == dk && state.size(3) == dv && powers.dim() == 2 &&
+                  powers.size(0) == H && powers.size(1) == 65 && cos_sin.dim() == 2 &&
+                  cos_sin.size(0) >= T && cos_sin.size(1) % 2 == 0 && cos_sin.size(1) <= dk &&
+                  num_decode >= 0 && num_decode <= S,
+              "retention: shapes");
+  const at::DeviceGuard g(v.device());
+  rc_ok(mixk_retention(out.data_ptr<float>(), state.data_ptr<float>(), q.data_ptr(), q.stride(0),
+                       k.data_ptr(), k.stride(0), v.data_ptr(), v.stride(0),
+                       powers.data_ptr<float>(), powers.size(1), cos_sin.data_ptr<float>(),
+                       cos_sin.size(1) / 2, positions.data_ptr<int>(), seq_qstart.data_ptr<int>(),
+                       seq_slot.data_ptr<int>(), S, num_decode, H, dk, dv, code(v), cur_stream()),
+        "retention");
 }
 
 void sigmoid_attention(at::Tensor out, const at::Tensor& q, const at::Tensor& k_cache,
@@ -490,18 +585,21 @@ void group_rms_norm(at::Tensor out, const at::Tensor& y, const c10::optional<at:
         "group_rms_norm");
 }
 
-void head_gate(at::Tensor out, const at::Tensor& o, const at::Tensor& gate) {
+void head_gate(at::Tensor out, const at::Tensor& o, const c10::optional<at::Tensor>& gate) {
   TORCH_CHECK(o.is_cuda() && o.dim() == 3 && o.is_contiguous(), "head_gate: o [H, T, dv]");
   const int64_t H = o.size(0), T = o.size(1), dv = o.size(2);
-  rows2d(gate, o, "gate");
-  // gate [T, H]: one number per head; [T, H * dv]: one per channel
-  TORCH_CHECK(gate.size(0) == T && (gate.size(1) == H || gate.size(1) == H * dv) &&
-                  out.is_contiguous() && out.numel() == o.numel() &&
+  TORCH_CHECK(out.is_contiguous() && out.numel() == o.numel() &&
                   out.scalar_type() == o.scalar_type(),
               "head_gate: shapes");
+  if (gate) {   // [T, H]: one number per head; [T, H * dv]: one per channel
+    rows2d(*gate, o, "gate");
+    TORCH_CHECK(gate->size(0) == T && (gate->size(1) == H || gate->size(1) == H * dv),
+                "head_gate: gate [T, H] or [T, H * dv]");
+  }
   const at::DeviceGuard g(o.device());
-  rc_ok(mixk_head_gate(out.data_ptr(), o.data_ptr(), gate.data_ptr(), gate.stride(0), T, H, dv,
-                       gate.size(1) != H, code(o), cur_stream()),
+  rc_ok(mixk_head_gate(out.data_ptr(), o.data_ptr(), gate ? gate->data_ptr() : nullptr,
+                       gate ? gate->stride(0) : 0, T, H, dv, gate && gate->size(1) != H, code(o),
+                       cur_stream()),
         "head_gate");
 }
 
@@ -710,7 +808,7 @@ void mingru_scan(at::Tensor out, at::Tensor state, const at::Tensor& z, const at
 
 void moe_route(at::Tensor idx, at::Tensor wts, const at::Tensor& logits, int64_t score,
                const c10::optional<at::Tensor>& correction, int64_t groups, int64_t keep,
-               bool renorm) {
+               bool renorm, double scale) {
   f32c(logits, "logits");
   if (correction) {
     f32c(*correction, "correction");
@@ -729,7 +827,8 @@ void moe_route(at::Tensor idx, at::Tensor wts, const at::Tensor& logits, int64_t
   const at::DeviceGuard g(logits.device());
   rc_ok(mixk_moe_route(idx.data_ptr<int>(), wts.data_ptr<float>(), logits.data_ptr<float>(),
                        correction ? correction->data_ptr<float>() : nullptr, logits.size(0),
-                       logits.size(1), idx.size(1), static_cast<int>(score), groups, keep, renorm, cur_stream()),
+                       logits.size(1), idx.size(1), static_cast<int>(score), groups, keep, renorm,
+                       static_cast<float>(scale), cur_stream()),
         "moe_route");
 }
 
@@ -781,18 +880,22 @@ void pair_sum(at::Tensor out, const at::Tensor& y) {
         "pair_sum");
 }
 
-void clamped_glu(at::Tensor out, const at::Tensor& gu, const at::Tensor& wts, double limit,
-                 double alpha) {
-  f32c(wts, "wts");
-  TORCH_CHECK(gu.is_cuda() && gu.dim() == 2 && gu.is_contiguous() && gu.size(1) % 2 == 0 &&
-                  out.is_cuda() && out.is_contiguous() && out.dim() == 2 &&
-                  out.size(0) == gu.size(0) && out.size(1) * 2 == gu.size(1) &&
-                  wts.numel() == gu.size(0) && out.scalar_type() == gu.scalar_type(),
-              "clamped_glu: gu [R, 2 ff], out [R, ff], wts [R]");
-  const at::DeviceGuard g(gu.device());
-  rc_ok(mixk_clamped_glu(out.data_ptr(), gu.data_ptr(), wts.data_ptr<float>(), gu.size(0),
+void clamped_glu(at::Tensor out, const at::Tensor& gate, const at::Tensor& up,
+                 const c10::optional<at::Tensor>& wts, double limit, double alpha) {
+  rows2d(gate, out, "gate");
+  rows2d(up, out, "up");
+  TORCH_CHECK(out.is_cuda() && out.is_contiguous() && out.dim() == 2 &&
+                  gate.sizes() == out.sizes() && up.sizes() == out.sizes(),
+              "clamped_glu: gate, up, out [R, ff]");
+  if (wts) {
+    f32c(*wts, "wts");
+    TORCH_CHECK(wts->numel() == out.size(0), "clamped_glu: wts [R]");
+  }
+  const at::DeviceGuard g(out.device());
+  rc_ok(mixk_clamped_glu(out.data_ptr(), gate.data_ptr(), gate.stride(0), up.data_ptr(),
+                         up.stride(0), wts ? wts->data_ptr<float>() : nullptr, out.size(0),
                          out.size(1), static_cast<float>(limit), static_cast<float>(alpha),
-                         code(gu), cur_stream()),
+                         code(out), cur_stream()),
         "clamped_glu");
 }
 
@@ -823,7 +926,8 @@ void moe_combine(at::Tensor out, const at::Tensor& y, const at::Tensor& idx, con
 
 void norm_add_norm(const c10::optional<at::Tensor>& h, at::Tensor x,
                    const c10::optional<at::Tensor>& y, const c10::optional<at::Tensor>& w_post,
-                   const c10::optional<at::Tensor>& w_next, double eps, bool layer) {
+                   const c10::optional<at::Tensor>& w_next,
+                   const c10::optional<at::Tensor>& post_scale, double eps, bool layer) {
   f32c(x, "x");
   TORCH_CHECK(x.dim() == 2 && (h.has_value() || y.has_value()) &&
                   h.has_value() == w_next.has_value() && y.has_value() == w_post.has_value(),
@@ -841,9 +945,14 @@ void norm_add_norm(const c10::optional<at::Tensor>& h, at::Tensor x,
   };
   if (h) { rows(*h); weight(*w_next); }
   if (y) { rows(*y); weight(*w_post); }
+  if (post_scale) {
+    TORCH_CHECK(y.has_value(), "norm_add_norm: post_scale goes with y");
+    weight(*post_scale);
+  }
   const at::DeviceGuard g(x.device());
   rc_ok(mixk_norm_add_norm(h ? h->data_ptr() : nullptr, x.data_ptr<float>(),
                            y ? y->data_ptr() : nullptr, w_post ? w_post->data_ptr() : nullptr,
+                           post_scale ? post_scale->data_ptr() : nullptr,
                            w_next ? w_next->data_ptr() : nullptr, x.size(0), x.size(1),
                            static_cast<float>(eps), layer, code(like), cur_stream()),
         "norm_add_norm");
@@ -910,7 +1019,7 @@ TORCH_LIBRARY(atta_mix, m) {
   m.def("residual_add(Tensor(a!) x, Tensor a, float sa, Tensor? b, float sb, Tensor? c) -> ()");
   m.def("add_norm(Tensor(a!) h, Tensor(b!) x, Tensor a, float sa, Tensor? b, float sb, Tensor? c, "
         "Tensor w, float eps, bool one_plus) -> ()");
-  m.def("gated_rms_norm(Tensor(a!) out, Tensor o, Tensor gate, Tensor w, float eps, int act) -> ()");
+  m.def("gated_rms_norm(Tensor(a!) out, Tensor o, Tensor gate, Tensor? w, float eps, int act) -> ()");
   m.def("qk_norm_rope_cache(Tensor(a!) q_out, Tensor qx, Tensor kx, Tensor vx, Tensor? q_norm, "
         "Tensor? k_norm, float eps, Tensor positions, Tensor slot_mapping, Tensor cos_sin, "
         "Tensor(b!) k_cache, Tensor(c!) v_cache, bool rotate_half, bool norm_last, "
@@ -920,7 +1029,15 @@ TORCH_LIBRARY(atta_mix, m) {
   m.def("sink_attention(Tensor(a!) out, Tensor q, Tensor k_cache, Tensor v_cache, "
         "Tensor block_tables, Tensor seq_kvlen, Tensor seq_qstart, Tensor tile_seq, "
         "Tensor tile_qoff, float scale, bool sink, int num_decode, int max_decode_kv, "
-        "Tensor? part, bool use_mfma, Tensor? sink_val, int window, Tensor? gate) -> ()");
+        "Tensor? part, bool use_mfma, Tensor? sink_val, int window, Tensor? gate, int keep, "
+        "float[]? pair) -> ()");
+  m.def("kv_cache_write(Tensor kx, Tensor vx, Tensor slot_mapping, Tensor(a!) k_cache, "
+        "Tensor(b!) v_cache) -> ()");
+  m.def("diff_combine(Tensor(a!) out, Tensor a, Tensor? gate, float lam, float diff, float eps, "
+        "int kv_heads) -> ()");
+  m.def("retention(Tensor(a!) out, Tensor(b!) state, Tensor q, Tensor k, Tensor v, Tensor powers, "
+        "Tensor cos_sin, Tensor positions, Tensor seq_qstart, Tensor seq_slot, int H, int dk, "
+        "int dv, int num_decode) -> ()");
   m.def("sigmoid_attention(Tensor(a!) out, Tensor q, Tensor k_cache, Tensor v_cache, "
         "Tensor block_tables, Tensor seq_kvlen, Tensor seq_qstart, Tensor tile_seq, "
         "Tensor tile_qoff, float scale, float cap, Tensor bias, Tensor talk, int num_decode, "
@@ -935,7 +1052,7 @@ TORCH_LIBRARY(atta_mix, m) {
   m.def("xielu_bias(Tensor(a!) out, Tensor x, Tensor? bias, float ap, float aq) -> ()");
   m.def("group_rms_norm(Tensor(a!) out, Tensor y, Tensor? gate, Tensor w, int n_groups, float eps) "
         "-> ()");
-  m.def("head_gate(Tensor(a!) out, Tensor o, Tensor gate) -> ()");
+  m.def("head_gate(Tensor(a!) out, Tensor o, Tensor? gate) -> ()");
   m.def("latent_rope_cache(Tensor(a!) q_out, Tensor q_lat, Tensor qx, Tensor? kvx, Tensor? c_norm, "
         "float eps, Tensor slot_mapping, Tensor cos_sin, Tensor(b!) k_cache, Tensor(c!) v_cache, "
         "Tensor(d!) c_out, bool rotate_half) -> ()");
@@ -951,16 +1068,17 @@ TORCH_LIBRARY(atta_mix, m) {
   m.def("mingru_scan(Tensor(a!) out, Tensor(b!) state, Tensor z, Tensor x, Tensor g, "
         "Tensor positions, Tensor seq_qstart, Tensor seq_slot) -> ()");
   m.def("pair_sum(Tensor(a!) out, Tensor y) -> ()");
-  m.def("clamped_glu(Tensor(a!) out, Tensor gu, Tensor wts, float limit, float alpha) -> ()");
+  m.def("clamped_glu(Tensor(a!) out, Tensor gate, Tensor up, Tensor? wts, float limit, float alpha) "
+        "-> ()");
   m.def("moe_route(Tensor(a!) idx, Tensor(b!) wts, Tensor logits, int score, Tensor? correction, "
-        "int groups, int keep, bool renorm) -> ()");
+        "int groups, int keep, bool renorm, float scale) -> ()");
   m.def("moe_experts(Tensor(a!) y, Tensor(b!) act, Tensor(c!) plan, Tensor h, Tensor idx, "
         "Tensor wts, Tensor w_gate, Tensor w_up, Tensor w_down, float limit, float alpha, "
         "int max_tiles, int tile_rows, int split, int glu) -> ()");
   m.def("moe_combine(Tensor(a!) out, Tensor y, Tensor idx, Tensor wts, Tensor h, Tensor? addend, "
         "int E, int split) -> ()");
   m.def("norm_add_norm(Tensor(a!)? h, Tensor(b!) x, Tensor? y, Tensor? w_post, Tensor? w_next, "
-        "float eps, bool layer) -> ()");
+        "Tensor? post_scale, float eps, bool layer) -> ()");
   m.def("post_norm(Tensor(a!)? h, Tensor(b!) x, float alpha, Tensor a, float sa, Tensor? b, "
         "float sb, Tensor w, float eps) -> ()");
   m.def("proj_inv_rms(Tensor(a!) out, Tensor qx, Tensor kx, float eps) -> ()");
@@ -977,6 +1095,9 @@ TORCH_LIBRARY_IMPL(atta_mix, CUDA, m) {
   m.impl("qk_norm_rope_cache", &qk_norm_rope_cache);
   m.impl("rotary_table", &rotary_table);
   m.impl("sink_attention", &sink_attention);
+  m.impl("kv_cache_write", &kv_cache_write);
+  m.impl("diff_combine", &diff_combine);
+  m.impl("retention", &retention);
   m.impl("sigmoid_attention", &sigmoid_attention);
   m.impl("short_conv_silu", &short_conv_silu);
   m.impl("gated_delta_rule", &gated_delta_rule);

@@ -188,7 +188,7 @@ __global__ void add_norm_kernel(T* __restrict__ h, float* __restrict__ x, const 
     stf(h + base + i, x[base + i] * inv * (ldf(w + i) + plus));
 }
 
-// One wave per (row, head): o / sqrt(mean(o^2) + eps) * w * act(gate).
+// One wave per (row, head): o / sqrt(mean(o^2) + eps) * w * act(gate); w nullptr: no weight.
 template <typename T>
 __global__ void gated_rms_norm_kernel(T* __restrict__ out, const float* __restrict__ o,
                                       const T* __restrict__ gate, int64_t gate_stride,
@@ -204,10 +204,44 @@ __global__ void gated_rms_norm_kernel(T* __restrict__ out, const float* __restri
   for (int i = threadIdx.x; i < dv; i += kWave) {
     const float gv = ldf(g + i);
     const float ga = act == 1 ? sigmoidf_(gv) : siluf_(gv);
-    stf(y + i, orow[i] * inv * ldf(w + i) * ga);
+    stf(y + i, orow[i] * inv * (w != nullptr ? ldf(w + i) : 1.0f) * ga);
   }
 }
 
+// The same with 8 channels per lane (dv % 8 == 0, dv <= 8 LPR, aligned rows): LPR lanes per
+// (row, head), so a wave holds 64 / LPR of them and a workgroup four waves' worth.
+template <typename T, int LPR>
+__global__ void __launch_bounds__(256)
+gated_rms_norm_vec_kernel(T* __restrict__ out, const float* __restrict__ o,
+                          const T* __restrict__ gate, int64_t gate_stride, const T* __restrict__ w,
+                          int64_t items, int H, int dv, float eps, int act) {
+  const int64_t item = static_cast<int64_t>(blockIdx.x) * (256 / LPR) + threadIdx.x / LPR;
+  const int i = (threadIdx.x % LPR) * 8;
+  const bool on = item < items && i < dv;
+  const int64_t t = on ? item / H : 0;
+  const int h = static_cast<int>(on ? item % H : 0);
+  float v[8], gv[8];
+  float ss = 0.f;
+  if (on) {
+    ld8(o + item * dv + i, v);
+    ld8(gate + t * gate_stride + static_cast<int64_t>(h) * dv + i, gv);
+#pragma unroll
+    for (int e = 0; e < 8; ++e) ss += v[e] * v[e];
+  }
+#pragma unroll
+  for (int k = LPR / 2; k > 0; k >>= 1) ss += __shfl_xor(ss, k, kWave);
+  if (!on) return;
+  const float inv = 1.0f / sqrtf(ss / static_cast<float>(dv) + eps);
+#pragma unroll
+  for (int e = 0; e < 8; ++e) v[e] *= inv * (act == 1 ? sigmoidf_(gv[e]) : siluf_(gv[e]));
+  if (w != nullptr) {
+    float wv[8];
+    ld8(w + i, wv);
+#pragma unroll
+    for (int e = 0; e < 8; ++e) v[e] *= wv[e];
+  }
+  st8(out + item * dv + i, v);
+}
 
 // Token embedding times a constant into the fp32 residual stream, `copies` times per row (the
 // streams of a multi-stream residual all start as the embedding); one block per row.
@@ -351,7 +385,7 @@ __global__ void group_rms_norm_vec_kernel(T* __restrict__ out, const float* __re
 }
 
 // Per-head sigmoid output gate with the head-major to row-major move:
-// out[t, h, :] = o[h, t, :] * sigmoid(gate[t, h]).
+// out[t, h, :] = o[h, t, :] * sigmoid(gate[t, h]) (gate nullptr: the move alone).
 template <typename T>
 __global__ void head_gate_kernel(T* __restrict__ out, const T* __restrict__ o,
                                  const T* __restrict__ gate, int64_t gate_stride, int T_, int H,
@@ -359,7 +393,8 @@ __global__ void head_gate_kernel(T* __restrict__ out, const T* __restrict__ o,
   const int t = blockIdx.x;
   for (int i = threadIdx.x; i < H * dv; i += blockDim.x) {
     const int h = i / dv, j = i - h * dv;
-    const float gv = sigmoidf_(ldf(gate + t * gate_stride + (per_channel ? i : h)));
+    const float gv = gate != nullptr
+                         ? sigmoidf_(ldf(gate + t * gate_stride + (per_channel ? i : h))) : 1.0f;
     stf(out + static_cast<int64_t>(t) * H * dv + i,
         ldf(o + (static_cast<int64_t>(h) * T_ + t) * dv + j) * gv);
   }
@@ -375,7 +410,8 @@ __global__ void head_gate_vec_kernel(T* __restrict__ out, const T* __restrict__ 
     const int h = i / dv, j = i - h * dv;
     float v[8], g[8];
     ld8(o + (static_cast<int64_t>(h) * T_ + t) * dv + j, v);
-    if (per_channel) {
+    if (gate == nullptr) {   // the move alone
+    } else if (per_channel) {
       ld8(gate + t * gate_stride + i, g);
 #pragma unroll
       for (int e = 0; e < 8; ++e) v[e] *= sigmoidf_(g[e]);
@@ -475,10 +511,30 @@ extern "C" int mixk_gated_rms_norm(void* out, const float* o, const void* gate,
                                    int64_t gate_stride, const void* w, int T_, int H, int dv,
                                    float eps, int act, int dtype, hipStream_t st) {
   if (T_ <= 0) return 0;
-  MIXK_DISPATCH(dtype, hipLaunchKernelGGL(gated_rms_norm_kernel<T>, dim3(T_ * H), dim3(kWave), 0,
-                                          st, static_cast<T*>(out), o,
-                                          static_cast<const T*>(gate), gate_stride,
-                                          static_cast<const T*>(w), H, dv, eps, act));
+  const uintptr_t mask = dtype == 2 ? 31 : 15;
+  const int64_t items = static_cast<int64_t>(T_) * H;
+  const bool vec = dv % 8 == 0 && dv <= 512 && gate_stride % 8 == 0 &&
+                   ((reinterpret_cast<uintptr_t>(out) | reinterpret_cast<uintptr_t>(gate) |
+                     reinterpret_cast<uintptr_t>(w)) & mask) == 0 &&
+                   (reinterpret_cast<uintptr_t>(o) & 31) == 0;
+#define MIXK_GRN(LPR)                                                                             \
+  hipLaunchKernelGGL((gated_rms_norm_vec_kernel<T, LPR>),                                         \
+                     dim3(static_cast<unsigned>((items + 256 / LPR - 1) / (256 / LPR))),          \
+                     dim3(256), 0, st, static_cast<T*>(out), o, static_cast<const T*>(gate),      \
+                     gate_stride, static_cast<const T*>(w), items, H, dv, eps, act)
+  MIXK_DISPATCH(dtype, {
+    if (vec && dv <= 64)
+      MIXK_GRN(8);
+    else if (vec && dv <= 128)
+      MIXK_GRN(16);
+    else if (vec)
+      MIXK_GRN(64);
+    else
+      hipLaunchKernelGGL(gated_rms_norm_kernel<T>, dim3(T_ * H), dim3(kWave), 0, st,
+                         static_cast<T*>(out), o, static_cast<const T*>(gate), gate_stride,
+                         static_cast<const T*>(w), H, dv, eps, act);
+  });
+#undef MIXK_GRN
   return static_cast<int>(hipGetLastError());
 }
 

@@ -36,9 +36,21 @@ int mixk_sink_attention(void* out, const void* q, const void* k_cache, const voi
                         const int* seq_qstart, const int* tile_seq, const int* tile_qoff,
                         int num_tiles, int num_decode, int max_decode_kv, float* part,
                         int max_parts, int H, int G, int dim, int vdim, int block_size,
-                        float scale, int sink, const float* sink_val, int window,
-                        const void* gate, int64_t gate_stride, int use_mfma, int dtype,
-                        hipStream_t st);
+                        float scale, int sink, const float* sink_val, int window, int keep,
+                        const void* gate, int64_t gate_stride, int v_share, int64_t q_stride,
+                        int out_f32, int pair, float lam, float post, float eps, int use_mfma,
+                        int dtype, hipStream_t st);
+int mixk_diff_combine(void* out, const float* in, const void* gate, int64_t gate_stride, int T,
+                      int HO, int G, int vdim, float lam, float post, float eps, int dtype,
+                      hipStream_t st);
+int mixk_kv_cache_write(const void* kx, int64_t k_stride, const void* vx, int64_t v_stride,
+                        const int* slot_mapping, void* k_cache, void* v_cache, int T, int GK,
+                        int dim, int GV, int vdim, int block_size, int dtype, hipStream_t st);
+int mixk_retention(float* out, float* state, const void* q, int64_t q_stride, const void* k,
+                   int64_t k_stride, const void* v, int64_t v_stride, const float* powers,
+                   int n_powers, const float* cos_sin, int n_freq, const int* positions,
+                   const int* seq_qstart, const int* seq_slot, int S, int num_decode, int H,
+                   int dk, int dv, int dtype, hipStream_t st);
 int mixk_sigmoid_attention(void* out, const void* q, const void* k_cache, const void* v_cache,
                            const int* block_tables, int bt_width, const int* seq_kvlen,
                            const int* seq_qstart, const int* tile_seq, const int* tile_qoff,
@@ -93,12 +105,14 @@ int mixk_mingru_scan(void* out, float* state, const void* z, int64_t z_stride, c
                      int64_t x_stride, const void* g, int64_t g_stride, const int* positions,
                      const int* seq_qstart, const int* seq_slot, int S, int C, int few_rows,
                      int dtype, hipStream_t st);
-int mixk_clamped_glu(void* out, const void* gu, const float* wts, int R, int ff, float limit,
-                     float alpha, int dtype, hipStream_t st);
+int mixk_clamped_glu(void* out, const void* gate, int64_t gate_stride, const void* up,
+                     int64_t up_stride, const float* wts, int R, int ff, float limit, float alpha,
+                     int dtype, hipStream_t st);
 int mixk_pair_sum(void* out, const void* y, int y_f32, int T, int top, int W, int dtype,
                   hipStream_t st);
 int mixk_moe_route(int* idx, float* wts, const float* logits, const float* correction, int T,
-                   int E, int top, int score, int groups, int keep, int renorm, hipStream_t st);
+                   int E, int top, int score, int groups, int keep, int renorm, float scale,
+                   hipStream_t st);
 int mixk_moe_experts(void* y, void* act, int* plan, const void* h, const int* idx,
                      const float* wts, const void* w_gate, const void* w_up, const void* w_down,
                      int T, int top, int E, int ff, int W, int64_t gu_estride, int max_tiles,
@@ -107,8 +121,9 @@ int mixk_moe_experts(void* y, void* act, int* plan, const void* h, const int* id
 int mixk_moe_combine(void* out, const void* y, int y_f32, const int* idx, const float* wts,
                      const void* h, const void* addend, int T, int top, int split, int E, int W,
                      int dtype, hipStream_t st);
-int mixk_norm_add_norm(void* h, float* x, const void* y, const void* w_post, const void* w_next,
-                       int T, int W, float eps, int layer, int dtype, hipStream_t st);
+int mixk_norm_add_norm(void* h, float* x, const void* y, const void* w_post,
+                       const void* post_scale, const void* w_next, int T, int W, float eps,
+                       int layer, int dtype, hipStream_t st);
 int mixk_post_norm(void* h, float* x, float alpha, const void* a, float sa, const void* b,
                    float sb, const void* w, int T, int W, float eps, int dtype, hipStream_t st);
 int mixk_proj_inv_rms(float* out, const void* qx, int64_t q_stride, int nq, const void* kx,

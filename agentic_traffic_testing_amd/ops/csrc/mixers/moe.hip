@@ -8,7 +8,7 @@
 //   neighbouring experts) scores its largest choice score, `keep` rounds of wave-wide arg-max
 //   pick the groups whose experts stay eligible; `top` rounds of wave-wide arg-max over the
 //   eligible choice scores (ties: lowest index) give idx [T, top]; wts [T, top] are the plain
-//   scores of the chosen, optionally divided by their sum + 1e-20.
+//   scores of the chosen, optionally divided by their sum + 1e-20, times a constant.
 // * moe_plan (one workgroup): histogram of the P = T * top pairs over the experts, prefix sums,
 //   the tile table (expert, first sorted position, rows <= rows_per_tile), and the pairs scattered
 //   into expert order.  plan = [ntiles, 0, tile_expert[max_tiles], tile_start[max_tiles],
@@ -33,7 +33,7 @@
 //   LDS tiles of 64 rows x 64 features.
 //   With glu = 1 the first product's epilogue is the plain SiLU GLU, silu(acc_g) acc_u, without
 //   the router weight (moe_combine applies it to the expert's output).
-// * clamped_glu (rows of [gate | up] products from library GEMMs), pair_sum (a row's choices and
+// * clamped_glu (rows of gate and up products from library GEMMs), pair_sum (a row's choices and
 //   split partials added in fp32), moe_combine (out[t] = sum_j w[t, j] y[t, j] (+ addend[t]) in
 //   fp32, where an index >= E is an identity expert whose output is the row of h itself).
 #include "mix_common.h"
@@ -65,7 +65,7 @@ template <int PER>
 __global__ void __launch_bounds__(256)
 moe_route_kernel(int* __restrict__ idx, float* __restrict__ wts, const float* __restrict__ logits,
                  const float* __restrict__ correction, int T_, int E, int top, int score,
-                 int groups, int keep, int renorm) {
+                 int groups, int keep, int renorm, float scale) {
   __shared__ float s_choice[4][PER * kWave];
   __shared__ unsigned char s_kept[4][PER * kWave];
   const int wv = threadIdx.x >> 6, lane = threadIdx.x & 63;
@@ -191,7 +191,7 @@ moe_route_kernel(int* __restrict__ idx, float* __restrict__ wts, const float* __
   for (int j = 0; j < PER; ++j)
     if (pick[j] >= 0) {
       idx[static_cast<int64_t>(t) * top + pick[j]] = lane + j * kWave;
-      wts[static_cast<int64_t>(t) * top + pick[j]] = norm ? sc[j] / (tot + 1e-20f) : sc[j];
+      wts[static_cast<int64_t>(t) * top + pick[j]] = (norm ? sc[j] / (tot + 1e-20f) : sc[j]) * scale;
     }
 }
 
@@ -486,17 +486,29 @@ moe_gemm_rows_kernel(T* __restrict__ out, const T* __restrict__ x, const T* __re
   }
 }
 
-// Clamped GLU over rows of [gate | up] products (the library path of prefill-sized steps): one
-// thread per output element, the row's router weight applied to both products first.
-template <typename T>
-__global__ void clamped_glu_kernel(T* __restrict__ out, const T* __restrict__ gu,
+// Clamped GLU over rows of gate and up products (a library product's column slices): the router
+// weight of the row (wts, nullptr: none) is applied to both products first.
+template <typename T, bool VEC>
+__global__ void clamped_glu_kernel(T* __restrict__ out, const T* __restrict__ gate,
+                                   int64_t gate_stride, const T* __restrict__ up, int64_t up_stride,
                                    const float* __restrict__ wts, int ff, float limit,
                                    float alpha) {
-  const int f = blockIdx.y * blockDim.x + threadIdx.x;
+  constexpr int N = VEC ? 8 : 1;
+  const int f = (blockIdx.y * blockDim.x + threadIdx.x) * N;
   if (f >= ff) return;
   const int64_t r = blockIdx.x;
-  const T* row = gu + r * 2 * ff;
-  stf(out + r * ff + f, clamped_glu(ldf(row + f), ldf(row + ff + f), wts[r], limit, alpha));
+  const float wt = wts != nullptr ? wts[r] : 1.0f;
+  float g[N], u[N];
+  if (VEC) {
+    ld8(gate + r * gate_stride + f, g);
+    ld8(up + r * up_stride + f, u);
+  } else {
+    g[0] = ldf(gate + r * gate_stride + f);
+    u[0] = ldf(up + r * up_stride + f);
+  }
+#pragma unroll
+  for (int e = 0; e < N; ++e) g[e] = clamped_glu(g[e], u[e], wt, limit, alpha);
+  if (VEC) st8(out + r * ff + f, g); else stf(out + r * ff + f, g[0]);
 }
 
 // out[t] = sum_j y[t, j] over a row's `top` summands, accumulated in fp32 in the order of j.
@@ -624,18 +636,31 @@ extern "C" int mixk_pair_sum(void* out, const void* y, int y_f32, int T_, int to
   return static_cast<int>(hipGetLastError());
 }
 
-extern "C" int mixk_clamped_glu(void* out, const void* gu, const float* wts, int R, int ff,
-                                float limit, float alpha, int dtype, hipStream_t st) {
+extern "C" int mixk_clamped_glu(void* out, const void* gate, int64_t gate_stride, const void* up,
+                                int64_t up_stride, const float* wts, int R, int ff, float limit,
+                                float alpha, int dtype, hipStream_t st) {
   if (R <= 0 || ff <= 0) return 0;
-  MIXK_DISPATCH(dtype, hipLaunchKernelGGL(clamped_glu_kernel<T>, dim3(R, (ff + 255) / 256),
-                                          dim3(256), 0, st, static_cast<T*>(out),
-                                          static_cast<const T*>(gu), wts, ff, limit, alpha));
+  const uintptr_t mask = dtype == 2 ? 31 : 15;
+  const bool vec = ff % 8 == 0 && gate_stride % 8 == 0 && up_stride % 8 == 0 &&
+                   ((reinterpret_cast<uintptr_t>(out) | reinterpret_cast<uintptr_t>(gate) |
+                     reinterpret_cast<uintptr_t>(up)) & mask) == 0;
+#define MIXK_CGLU(VEC)                                                                            \
+  hipLaunchKernelGGL((clamped_glu_kernel<T, VEC>), dim3(R, ((VEC ? ff / 8 : ff) + 255) / 256),    \
+                     dim3(256), 0, st, static_cast<T*>(out), static_cast<const T*>(gate),         \
+                     gate_stride, static_cast<const T*>(up), up_stride, wts, ff, limit, alpha)
+  MIXK_DISPATCH(dtype, {
+    if (vec)
+      MIXK_CGLU(true);
+    else
+      MIXK_CGLU(false);
+  });
+#undef MIXK_CGLU
   return static_cast<int>(hipGetLastError());
 }
 
 extern "C" int mixk_moe_route(int* idx, float* wts, const float* logits, const float* correction,
                               int T_, int E, int top, int score, int groups, int keep,
-                              int renorm, hipStream_t st) {
+                              int renorm, float scale, hipStream_t st) {
   if (T_ <= 0) return 0;
   if (score < kScoreSigmoid || score > kScoreLogit) return -1;
   if (E < 1 || E > kMaxExperts || top < 1 || top > E || groups < 1 || E % groups != 0 ||
@@ -643,7 +668,7 @@ extern "C" int mixk_moe_route(int* idx, float* wts, const float* logits, const f
     return -1;
 #define MIXK_ROUTE(PER)                                                                          \
   hipLaunchKernelGGL(moe_route_kernel<PER>, dim3((T_ + 3) / 4), dim3(256), 0, st, idx, wts,      \
-                     logits, correction, T_, E, top, score, groups, keep, renorm)
+                     logits, correction, T_, E, top, score, groups, keep, renorm, scale)
   if (E <= kWave)
     MIXK_ROUTE(1);
   else if (E <= 4 * kWave)

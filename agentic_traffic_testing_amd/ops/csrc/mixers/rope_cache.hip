@@ -191,6 +191,29 @@ __global__ void v_cache_write_kernel(const T* __restrict__ vx, int64_t v_stride,
   }
 }
 
+// K rows [T, GK * dim] as they are into the pages k_cache [nb, GK, BS, dim]: eight channels per
+// thread where widths and addresses allow (VEC), one otherwise.
+template <typename T, bool VEC>
+__global__ void k_cache_write_kernel(const T* __restrict__ kx, int64_t k_stride,
+                                     const int* __restrict__ slot_mapping, T* __restrict__ k_cache,
+                                     int GK, int dim, int block_size) {
+  constexpr int N = VEC ? 8 : 1;
+  const int64_t t = blockIdx.x;
+  const int i = (blockIdx.y * blockDim.x + threadIdx.x) * N;
+  const int slot = slot_mapping[t];
+  if (slot < 0 || i >= GK * dim) return;
+  const int g = i / dim, d = i - g * dim;
+  T* dst = k_cache + ((static_cast<int64_t>(slot / block_size) * GK + g) * block_size +
+                      slot % block_size) * dim + d;
+  const T* src = kx + t * k_stride + i;
+  if (VEC) {
+    float v[8];
+    ld8(src, v);
+    st8(dst, v);
+  } else {
+    *dst = *src;
+  }
+}
 
 // Latent attention front end (one shared key / value head of compressed rows): per row, one wave
 // per query head assembles the absorbed query [q_lat | rotated q_rot] and one more wave norms
@@ -337,5 +360,33 @@ extern "C" int mixk_latent_rope_cache(void* q_out, const void* q_lat, const void
                          static_cast<T*>(v_cache), T_, 1, rank, block_size, ValueArgs{0.f, 0.f, 0},
                          static_cast<const T*>(nullptr), static_cast<T*>(nullptr));
   });
+  return static_cast<int>(hipGetLastError());
+}
+
+extern "C" int mixk_kv_cache_write(const void* kx, int64_t k_stride, const void* vx,
+                                   int64_t v_stride, const int* slot_mapping, void* k_cache,
+                                   void* v_cache, int T_, int GK, int dim, int GV, int vdim,
+                                   int block_size, int dtype, hipStream_t st) {
+  if (T_ <= 0) return 0;
+  if (GK <= 0 || GV <= 0 || dim <= 0 || vdim <= 0 || block_size <= 0) return -1;
+  const uintptr_t mask = dtype == 2 ? 31 : 15;
+  const bool vec = dim % 8 == 0 && k_stride % 8 == 0 &&
+                   ((reinterpret_cast<uintptr_t>(kx) | reinterpret_cast<uintptr_t>(k_cache)) & mask) == 0;
+  const int n = GK * dim;
+#define MIXK_KW(VEC)                                                                               \
+  hipLaunchKernelGGL((k_cache_write_kernel<T, VEC>), dim3(T_, ((VEC ? n / 8 : n) + 127) / 128),    \
+                     dim3(128), 0, st, static_cast<const T*>(kx), k_stride, slot_mapping,          \
+                     static_cast<T*>(k_cache), GK, dim, block_size)
+  MIXK_DISPATCH(dtype, {
+    if (vec)
+      MIXK_KW(true);
+    else
+      MIXK_KW(false);
+    hipLaunchKernelGGL((v_cache_write_kernel<T, false>), dim3((T_ + 7) / 8, GV), dim3(128), 0, st,
+                       static_cast<const T*>(vx), v_stride, slot_mapping, static_cast<T*>(v_cache),
+                       T_, GV, vdim, block_size, ValueArgs{0.f, 0.f, 0},
+                       static_cast<const T*>(nullptr), static_cast<T*>(nullptr));
+  });
+#undef MIXK_KW
   return static_cast<int>(hipGetLastError());
 }

@@ -5,7 +5,7 @@
 //     x = rms(alpha x + sa a [+ sb b]) * w    (fp32, in place)
 //   and h, when given, takes the new x in the activation dtype - what the next sub-layer reads.
 // * norm_add_norm: one workgroup per row of the fp32 residual x [T, W]:
-//     x += norm(y) * w_post          (skipped when y is nullptr)
+//     x += norm(y) * w_post [* post_scale]   (skipped when y is nullptr)
 //     h  = norm(x) * w_next          (skipped when h is nullptr)
 //   norm = layer norm without bias, (v - mean) / sqrt(var + eps) with var the mean squared
 //   deviation (two passes over registers: the mean first, then the deviations), or RMS norm,
@@ -52,6 +52,7 @@ __device__ __forceinline__ void row_stats(float (&v)[kSwGroups][8], int W, float
 template <typename T, bool LAYER>
 __global__ void norm_add_norm_vec_kernel(T* __restrict__ h, float* __restrict__ x,
                                          const T* __restrict__ y, const T* __restrict__ w_post,
+                                         const T* __restrict__ post_scale,
                                          const T* __restrict__ w_next, int W, float eps) {
   __shared__ float scratch[16];
   const int64_t base = static_cast<int64_t>(blockIdx.x) * W;
@@ -73,6 +74,12 @@ __global__ void norm_add_norm_vec_kernel(T* __restrict__ h, float* __restrict__ 
       if (i < W) {
         float wv[8];
         ld8(w_post + i, wv);
+        if (post_scale != nullptr) {
+          float sv[8];
+          ld8(post_scale + i, sv);
+#pragma unroll
+          for (int e = 0; e < 8; ++e) wv[e] *= sv[e];
+        }
 #pragma unroll
         for (int e = 0; e < 8; ++e) xv[g][e] += (yv[g][e] - mean) * inv * wv[e];
         st8(x + base + i, xv[g]);
@@ -99,6 +106,7 @@ __global__ void norm_add_norm_vec_kernel(T* __restrict__ h, float* __restrict__ 
 template <typename T, bool LAYER>
 __global__ void norm_add_norm_kernel(T* __restrict__ h, float* __restrict__ x,
                                      const T* __restrict__ y, const T* __restrict__ w_post,
+                                     const T* __restrict__ post_scale,
                                      const T* __restrict__ w_next, int W, float eps) {
   __shared__ float scratch[16];
   const int64_t base = static_cast<int64_t>(blockIdx.x) * W;
@@ -118,7 +126,8 @@ __global__ void norm_add_norm_kernel(T* __restrict__ h, float* __restrict__ x,
     }
     const float inv = 1.0f / sqrtf(block_sum(ss, scratch) / static_cast<float>(W) + eps);
     for (int i = threadIdx.x; i < W; i += blockDim.x)
-      xr[i] += (ldf(yr + i) - mean) * inv * ldf(w_post + i);
+      xr[i] += (ldf(yr + i) - mean) * inv *
+               (ldf(w_post + i) * (post_scale != nullptr ? ldf(post_scale + i) : 1.0f));
   }
   if (h == nullptr) return;
   float mean = 0.f;
@@ -260,21 +269,22 @@ static bool al32(const void* p) { return (reinterpret_cast<uintptr_t>(p) & 31) =
 using namespace mixk;
 
 extern "C" int mixk_norm_add_norm(void* h, float* x, const void* y, const void* w_post,
-                                  const void* w_next, int T_, int W, float eps, int layer,
-                                  int dtype, hipStream_t st) {
+                                  const void* post_scale, const void* w_next, int T_, int W,
+                                  float eps, int layer, int dtype, hipStream_t st) {
   if (T_ <= 0 || W <= 0) return 0;
   if ((y != nullptr && w_post == nullptr) || (h != nullptr && w_next == nullptr)) return -1;
   int threads = sandwich_threads(W);
   // 16-byte loads of the activation rows, 32-byte pairs of the fp32 residual
   if (!(al32(x) && (h == nullptr || al16(h)) && (y == nullptr || al16(y)) &&
-        (w_post == nullptr || al16(w_post)) && (w_next == nullptr || al16(w_next))) ||
+        (w_post == nullptr || al16(w_post)) && (post_scale == nullptr || al16(post_scale)) && (w_next == nullptr || al16(w_next))) ||
       (dtype == 2 && !((h == nullptr || al32(h)) && (y == nullptr || al32(y)) &&
-                       (w_post == nullptr || al32(w_post)) && (w_next == nullptr || al32(w_next)))))
+                       (w_post == nullptr || al32(w_post)) &&
+                       (post_scale == nullptr || al32(post_scale)) && (w_next == nullptr || al32(w_next)))))
     threads = 0;
 #define MIXK_SANDWICH(KERNEL, LAYER, THREADS)                                                    \
   hipLaunchKernelGGL((KERNEL<T, LAYER>), dim3(T_), dim3(THREADS), 0, st, static_cast<T*>(h), x,  \
                      static_cast<const T*>(y), static_cast<const T*>(w_post),                    \
-                     static_cast<const T*>(w_next), W, eps)
+                     static_cast<const T*>(post_scale), static_cast<const T*>(w_next), W, eps)
   MIXK_DISPATCH(dtype, {
     if (threads && layer)
       MIXK_SANDWICH(norm_add_norm_vec_kernel, true, threads);

@@ -26,6 +26,17 @@
 // touch its edge; decode then runs only the partitions that overlap the window (partition
 // indices are relative to the first of them, for the partition kernel and the combine alike).
 //
+// With `keep` > 0 the window also keeps a sequence's first `keep` keys: key tiles (or, in decode,
+// partitions) of the range [0, keep) that lie before the window run first, then the walk jumps to
+// the window; every mask is "not before the window, or among the first `keep`".
+//
+// A V head may serve `v_share` neighbouring K heads (the maps of differential attention).  In the
+// pair form (two maps per V head, heads in the order KV head, map, head of the group) a column of
+// the matrix-core prefill kernel carries both maps: two K tiles, two softmax states, two
+// accumulators over one staged V tile, and the epilogue a1 - lambda a2, its root mean square over
+// the head, the factor and the element-wise sigmoid gate; in decode the two maps are separate
+// workgroups and the pair form of the combine kernel joins them.
+//
 // A per-head output gate (`gate`) multiplies the result by sigmoid(gate[row, head]) in the kernel
 // that stores it.
 //
@@ -54,6 +65,12 @@ struct AttnArgs {
   int bt_width, H, G, dim, vdim, block_size, sink, KT, max_parts, bs_shift;
   float scale;
   int window;   // 0: every earlier key
+  int keep;     // with a window: the first keys stay visible
+  int v_share;  // K heads per V head
+  int64_t q_stride;   // elements between two rows of q
+  int out_f32;  // results are stored as fp32 whatever T
+  int pair;     // pair form: a1 - lam a2, then / rms (eps) * post, gate [T, H / 2 * vdim]
+  float lam, post, eps;
   const void* gate;       // row-strided [T, H] of the activation dtype, or nullptr: head h's output
   int64_t gate_stride;    // of row t is multiplied by sigmoid(gate[t, h])
 };
@@ -69,15 +86,28 @@ __device__ __forceinline__ int window_start(int qpos, int window) {
   return window > 0 ? max(0, qpos - window + 1) : 0;
 }
 
+// decode partitions that hold only kept keys, all in front of the window's first partition
+__device__ __forceinline__ int keep_parts(int keep, int wstart) {
+  return min((keep + kPartTokens - 1) / kPartTokens, wstart / kPartTokens);
+}
+
+template <typename T>
+__device__ __forceinline__ void st_out(void* out, int64_t i, float v, int out_f32) {
+  if (out_f32)
+    static_cast<float*>(out)[i] = v;
+  else
+    stf(static_cast<T*>(out) + i, v);
+}
+
 template <typename T, bool DECODE>
 __global__ void __launch_bounds__(256)
-sink_attention_rows_kernel(T* __restrict__ out, const T* __restrict__ q,
+sink_attention_rows_kernel(void* __restrict__ out, const T* __restrict__ q,
                            const T* __restrict__ k_cache, const T* __restrict__ v_cache,
                            AttnArgs a) {
   extern __shared__ float smem[];
   const int H = a.H, G = a.G, dim = a.dim, vdim = a.vdim, KT = a.KT, bs = a.block_size;
   const int rep = H / G;
-  int s, g, nrows, kbeg, kend, kvlen, n, row0, qo = 0, h0;
+  int s, g, nrows, kbeg, kend, kvlen, n, row0, qo = 0, h0, klo = 0;
   if (DECODE) {
     // blockIdx.y = (KV head, block of up to kRows query heads of its group)
     const int hb = (rep + kRows - 1) / kRows;
@@ -89,10 +119,11 @@ sink_attention_rows_kernel(T* __restrict__ out, const T* __restrict__ q,
     h0 = g * rep + (blockIdx.y % hb) * kRows;
     nrows = min(kRows, (g + 1) * rep - h0);
     if (kvlen <= 0) return;
-    const int wstart = window_start(kvlen - 1, a.window);
-    kbeg = (wstart / kPartTokens + blockIdx.z) * kPartTokens;
-    kend = min(kvlen, kbeg + kPartTokens);
-    kbeg = max(kbeg, wstart);
+    const int wstart = window_start(kvlen - 1, a.window), kp = keep_parts(a.keep, wstart);
+    const int z = blockIdx.z;
+    klo = z < kp ? z * kPartTokens : (wstart / kPartTokens + z - kp) * kPartTokens;
+    kend = min(z < kp ? a.keep : kvlen, klo + kPartTokens);
+    kbeg = z < kp ? klo : max(klo, wstart);
     if (kbeg >= kend) return;
   } else {
     const int tile = blockIdx.x >> 2;
@@ -120,7 +151,7 @@ sink_attention_rows_kernel(T* __restrict__ out, const T* __restrict__ q,
     if (rr < nrows) {
       const int64_t qrow = DECODE ? row0 : row0 + qo + rr;
       const int head = DECODE ? h0 + rr : h0;
-      v = ldf(q + (qrow * H + head) * dim + d);
+      v = ldf(q + qrow * a.q_stride + static_cast<int64_t>(head) * dim + d);
     }
     Qs[i] = v;
   }
@@ -138,13 +169,16 @@ sink_attention_rows_kernel(T* __restrict__ out, const T* __restrict__ q,
   for (int j = 0; j < kMaxVPer; ++j) acc[j] = 0.f;
   const int* bt = a.block_tables + static_cast<int64_t>(s) * a.bt_width;
   const int kper = KT >> 4;
-  for (int k0 = kbeg; k0 < kend; k0 += KT) {
+  // kept keys [klo, kkeep) in front of the window, then [kbeg, kend)
+  const int kkeep = min(a.keep, kbeg), gv = g / a.v_share, GV = G / a.v_share;
+  bool kept = klo < kkeep;
+  for (int k0 = kept ? klo : kbeg, te = kept ? kkeep : kend; k0 < kend;) {
     __syncthreads();  // previous tile fully consumed (and Qs written, first time round)
     for (int i = tid; i < KT * dim; i += 256) {
       const int kk = i / dim, d = i - kk * dim;
       const int tok = k0 + kk;
       float val = 0.f;
-      if (tok < kend) {
+      if (tok < te) {
         const int64_t page = bt[tok / bs];
         val = ldf(k_cache + ((page * G + g) * bs + tok % bs) * dim + d);
       }
@@ -154,9 +188,9 @@ sink_attention_rows_kernel(T* __restrict__ out, const T* __restrict__ q,
       const int d = i / KT, kk = i - d * KT;   // keys fastest: contiguous inside a page row
       const int tok = k0 + kk;
       float val = 0.f;
-      if (tok < kend) {
+      if (tok < te) {
         const int64_t page = bt[tok / bs];
-        val = ldf(v_cache + ((page * G + g) * vdim + d) * bs + tok % bs);
+        val = ldf(v_cache + ((page * GV + gv) * vdim + d) * bs + tok % bs);
       }
       Vs[kk * vstride + d] = val;
     }
@@ -171,7 +205,7 @@ sink_attention_rows_kernel(T* __restrict__ out, const T* __restrict__ q,
       if (row_ok)
         for (int d = 0; d < dim; ++d) dot += qr[d] * kr[d];
       const int tok = k0 + kk;
-      sc[j] = (row_ok && tok <= qpos && tok >= qlow && tok < kend) ? dot * a.scale : kNegBig;
+      sc[j] = (row_ok && tok <= qpos && (tok >= qlow || tok < a.keep) && tok < te) ? dot * a.scale : kNegBig;
       tmax = fmaxf(tmax, sc[j]);
     }
 #pragma unroll
@@ -199,6 +233,12 @@ sink_attention_rows_kernel(T* __restrict__ out, const T* __restrict__ q,
         acc[j] = av;
       }
     }
+    k0 += KT;
+    if (kept && k0 >= kkeep) {
+      kept = false;
+      k0 = kbeg;
+      te = kend;
+    }
   }
   if (!row_ok) return;
   if (DECODE) {
@@ -216,11 +256,11 @@ sink_attention_rows_kernel(T* __restrict__ out, const T* __restrict__ q,
     return;
   }
   const float inv = (l > 0.f ? 1.0f / l : 0.f) * head_gate_of<T>(a, row0 + qo + r, h0);
-  T* o = out + (static_cast<int64_t>(row0 + qo + r) * H + h0) * vdim;
+  const int64_t o = (static_cast<int64_t>(row0 + qo + r) * H + h0) * vdim;
 #pragma unroll
   for (int j = 0; j < kMaxVPer; ++j) {
     const int d = c + 16 * j;
-    if (d < vdim) stf(o + d, acc[j] * inv);
+    if (d < vdim) st_out<T>(out, o + d, acc[j] * inv, a.out_f32);
   }
 }
 
@@ -228,14 +268,19 @@ sink_attention_rows_kernel(T* __restrict__ out, const T* __restrict__ q,
 // fetches partition p's (m, l) (all in flight at once), the wave reduces them, and the
 // per-partition weights go through LDS for the channel loop.
 constexpr int kMaxParts = 2048;
+
+__device__ __forceinline__ int live_parts(const AttnArgs& a, int kvlen) {
+  const int wstart = window_start(kvlen - 1, a.window);
+  return (kvlen + kPartTokens - 1) / kPartTokens - wstart / kPartTokens + keep_parts(a.keep, wstart);
+}
+
 template <typename T>
-__global__ void sink_attention_combine_kernel(T* __restrict__ out, AttnArgs a) {
+__global__ void sink_attention_combine_kernel(void* __restrict__ out, AttnArgs a) {
   __shared__ float wts[kMaxParts];
   const int s = blockIdx.x, h = blockIdx.y, lane = threadIdx.x;
   const int kvlen = a.seq_kvlen[s];
   if (kvlen <= 0) return;
-  const int np = min(kMaxParts, (kvlen + kPartTokens - 1) / kPartTokens -
-                                    window_start(kvlen - 1, a.window) / kPartTokens);
+  const int np = min(kMaxParts, live_parts(a, kvlen));
   const int vdim = a.vdim, ps = vdim + 2;
   const float* base = a.part + (static_cast<int64_t>(s) * a.H + h) * a.max_parts * ps;
   const float sink_score = a.sink_val != nullptr ? a.sink_val[h] : 0.f;
@@ -252,13 +297,98 @@ __global__ void sink_attention_combine_kernel(T* __restrict__ out, AttnArgs a) {
   L = wave_sum(L) + (a.sink ? expf(sink_score - M) : 0.f);
   __syncthreads();
   const float inv = (L > 0.f ? 1.0f / L : 0.f) * head_gate_of<T>(a, a.seq_qstart[s], h);
-  T* o = out + (static_cast<int64_t>(a.seq_qstart[s]) * a.H + h) * vdim;
+  const int64_t o = (static_cast<int64_t>(a.seq_qstart[s]) * a.H + h) * vdim;
   for (int d = lane; d < vdim; d += kWave) {
     float v = 0.f;
 #pragma unroll 8
     for (int p = 0; p < np; ++p) v += base[p * ps + d] * wts[p];
-    stf(o + d, v * inv);
+    st_out<T>(out, o + d, v * inv, a.out_f32);
   }
+}
+
+// Pair form, one wave per (decode sequence, output head): merges the partitions of both maps, then
+// o = a1 - lam a2, / its root mean square, * post * sigmoid(gate per channel) into out [T, H / 2, vdim].
+template <typename T>
+__global__ void pair_attention_combine_kernel(T* __restrict__ out, AttnArgs a) {
+  __shared__ float wts[2][kMaxParts];
+  const int s = blockIdx.x, ho = blockIdx.y, lane = threadIdx.x;
+  const int kvlen = a.seq_kvlen[s];
+  if (kvlen <= 0) return;
+  const int rep = a.H / a.G, g = ho / rep;   // G counts a K head per map
+  const int np = min(kMaxParts, live_parts(a, kvlen));
+  const int vdim = a.vdim, ps = vdim + 2;
+  const float* base[2];
+  float inv[2];
+#pragma unroll
+  for (int mp = 0; mp < 2; ++mp) {
+    const int h = (2 * g + mp) * rep + ho % rep;
+    base[mp] = a.part + (static_cast<int64_t>(s) * a.H + h) * a.max_parts * ps;
+    float M = kNegBig, L = 0.f;
+    for (int p = lane; p < np; p += kWave) M = fmaxf(M, base[mp][p * ps + vdim]);
+#pragma unroll
+    for (int o = 32; o > 0; o >>= 1) M = fmaxf(M, __shfl_xor(M, o, kWave));
+    for (int p = lane; p < np; p += kWave) {
+      const float wp = expf(base[mp][p * ps + vdim] - M);
+      wts[mp][p] = wp;
+      L += base[mp][p * ps + vdim + 1] * wp;
+    }
+    L = wave_sum(L);
+    inv[mp] = L > 0.f ? 1.0f / L : 0.f;
+  }
+  __syncthreads();
+  constexpr int kPer = 16 * kMaxVPer / kWave;   // channels per lane
+  float o[kPer];
+  float ss = 0.f;
+#pragma unroll
+  for (int j = 0; j < kPer; ++j) {
+    const int d = lane + j * kWave;
+    o[j] = 0.f;
+    if (d < vdim) {
+      float v0 = 0.f, v1 = 0.f;
+#pragma unroll 4
+      for (int p = 0; p < np; ++p) {
+        v0 += base[0][p * ps + d] * wts[0][p];
+        v1 += base[1][p * ps + d] * wts[1][p];
+      }
+      o[j] = v0 * inv[0] - a.lam * (v1 * inv[1]);
+      ss += o[j] * o[j];
+    }
+  }
+  const float f = a.post / sqrtf(wave_sum(ss) / static_cast<float>(vdim) + a.eps);
+  const int64_t row = a.seq_qstart[s];
+  const T* gt = a.gate != nullptr ? static_cast<const T*>(a.gate) + row * a.gate_stride +
+                                        static_cast<int64_t>(ho) * vdim : nullptr;
+  T* orow = out + (row * (a.H / 2) + ho) * vdim;
+#pragma unroll
+  for (int j = 0; j < kPer; ++j) {
+    const int d = lane + j * kWave;
+    if (d < vdim) stf(orow + d, o[j] * f * (gt != nullptr ? sigmoidf_(ldf(gt + d)) : 1.0f));
+  }
+}
+
+// The same join over fp32 rows [T, H, vdim] of both maps (prefill without the matrix-core kernel):
+// one wave per (row, output head).
+template <typename T>
+__global__ void diff_combine_kernel(T* __restrict__ out, const float* __restrict__ in,
+                                    const T* __restrict__ gate, int64_t gate_stride, int T_, int HO,
+                                    int G, int vdim, float lam, float post, float eps) {
+  const int64_t idx = static_cast<int64_t>(blockIdx.x) * 4 + (threadIdx.x >> 6);
+  const int lane = threadIdx.x & 63;
+  if (idx >= static_cast<int64_t>(T_) * HO) return;
+  const int64_t t = idx / HO;
+  const int ho = static_cast<int>(idx % HO), rep = HO / G, g = ho / rep;
+  const float* a1 = in + (t * 2 * HO + 2 * g * rep + ho % rep) * vdim;
+  const float* a2 = a1 + static_cast<int64_t>(rep) * vdim;
+  float ss = 0.f;
+  for (int d = lane; d < vdim; d += kWave) {
+    const float o = a1[d] - lam * a2[d];
+    ss += o * o;
+  }
+  const float f = post / sqrtf(wave_sum(ss) / static_cast<float>(vdim) + eps);
+  const T* gt = gate != nullptr ? gate + t * gate_stride + static_cast<int64_t>(ho) * vdim : nullptr;
+  T* orow = out + (t * HO + ho) * vdim;
+  for (int d = lane; d < vdim; d += kWave)
+    stf(orow + d, (a1[d] - lam * a2[d]) * f * (gt != nullptr ? sigmoidf_(ldf(gt + d)) : 1.0f));
 }
 
 // ---- matrix-core prefill (bf16) -----------------------------------------------------------
@@ -275,18 +405,20 @@ constexpr int kVStride = kKeys + 8;
 // query heads of the group for the sequence's single new token, the output is the partition's
 // partial (unnormalised sum, m, l) for the combine kernel.  Waves without a valid column only
 // help to stage the tiles.
-template <int ND, int NV, bool DECODE>  // dim <= 16 ND, vdim <= 32 NV
-__global__ void __launch_bounds__(256, 2)
-sink_attention_mfma_kernel(__bf16* __restrict__ out, const __bf16* __restrict__ q,
+// NMAP 2: the pair form (blockIdx.y is the V head; prefill only).
+template <int ND, int NV, bool DECODE, int NMAP = 1>  // dim <= 16 ND, vdim <= 32 NV
+__global__ void __launch_bounds__(256, NMAP == 2 && ND > 8 ? 1 : 2)
+sink_attention_mfma_kernel(void* __restrict__ out, const __bf16* __restrict__ q,
                            const __bf16* __restrict__ k_cache, const __bf16* __restrict__ v_cache,
                            AttnArgs a) {
   constexpr int KS = ND * 16 + 8;
-  __shared__ __attribute__((aligned(16))) __bf16 lds_k[kKeys * KS];
+  __shared__ __attribute__((aligned(16))) __bf16 lds_k[NMAP * kKeys * KS];
   __shared__ __attribute__((aligned(16))) __bf16 lds_v[NV * 32 * kVStride];
   __shared__ int lds_bt[kBtLds];
   const int H = a.H, G = a.G, dim = a.dim, vdim = a.vdim, bs = a.block_size;
   const int rep = H / G, nd = dim >> 4, nv = vdim >> 5;
-  const int g = blockIdx.y;
+  const int g = blockIdx.y;              // K head (NMAP 2: V head, K heads 2 g and 2 g + 1)
+  const int gv = NMAP == 2 ? g : g / a.v_share, GV = G / a.v_share;
   // tiles are listed in sequence order, so the ones with the most keys come last: start those
   // first (the tail of the launch is then made of short tiles)
   const int tile = DECODE ? 0 : static_cast<int>(gridDim.x - 1 - blockIdx.x);
@@ -305,18 +437,22 @@ sink_attention_mfma_kernel(__bf16* __restrict__ out, const __bf16* __restrict__ 
   const int col = col0 + w * 32 + r;
   const bool valid = col < cols_total;
   const int tok = valid ? col / rep : 0;
-  const int head = g * rep + (valid ? col % rep : 0);
+  const int head = NMAP * g * rep + (valid ? col % rep : 0);   // of the first map
   const int64_t qrow = row0 + qo + tok;
   const int qpos = kvlen - n + qo + tok;
   const int last_tok = (min(cols_total, col0 + 128) - 1) / rep;
   // first key tile: the window's start of the workgroup's earliest column, on a tile boundary
   // (the V^T staging reads 8 keys at a time from 8-aligned slots)
   const int wstart = window_start(kvlen - n + qo + col0 / rep, a.window);
-  const int part0 = DECODE ? (wstart / kPartTokens + blockIdx.z) * kPartTokens : 0;
-  const int kbeg = max(part0, wstart & ~(kKeys - 1));
-  const int kend = DECODE ? min(kvlen, part0 + kPartTokens)
+  const int kp = DECODE ? keep_parts(a.keep, wstart) : 0;
+  const bool keep_part = DECODE && static_cast<int>(blockIdx.z) < kp;   // kept keys only
+  const int part0 = !DECODE ? 0 : keep_part ? static_cast<int>(blockIdx.z) * kPartTokens
+                                            : (wstart / kPartTokens + static_cast<int>(blockIdx.z) - kp) * kPartTokens;
+  const int kbeg = keep_part ? part0 : max(part0, wstart & ~(kKeys - 1));
+  const int kend = DECODE ? min(keep_part ? a.keep : kvlen, part0 + kPartTokens)
                           : min(kvlen, kvlen - n + qo + last_tok + 1);
   if (kbeg >= kend) return;
+  const int kkeep = min(a.keep, kbeg);   // kept keys [part0, kkeep) in front of the window
   const bool wave_on = col0 + w * 32 < cols_total;   // wave-uniform
   const int qpos_first = kvlen - n + qo + (col0 + w * 32) / rep;   // the wave's earliest column
   // the wave's latest column: keys at or below its window start are outside somebody's window
@@ -325,24 +461,30 @@ sink_attention_mfma_kernel(__bf16* __restrict__ out, const __bf16* __restrict__ 
   const int qlow = window_start(qpos, a.window);
   const float scale2 = a.scale * 1.44269504088896341f;
   const bool use_sink = a.sink && !DECODE;           // decode: the combine kernel adds it once
-  bf16x8 qf[ND];
+  bf16x8 qf[NMAP][ND];
+  float m[NMAP], l[NMAP];
+  f32x16 O[NMAP][NV];
 #pragma unroll
-  for (int st = 0; st < ND; ++st) {
-    u32x4 z = {0u, 0u, 0u, 0u};
-    if (valid && st < nd)
-      z = *reinterpret_cast<const u32x4*>(q + (qrow * H + head) * dim + st * 16 + 8 * h);
-    qf[st] = __builtin_bit_cast(bf16x8, z);
+  for (int mp = 0; mp < NMAP; ++mp) {
+#pragma unroll
+    for (int st = 0; st < ND; ++st) {
+      u32x4 z = {0u, 0u, 0u, 0u};
+      if (valid && st < nd)
+        z = *reinterpret_cast<const u32x4*>(q + qrow * a.q_stride +
+                                            static_cast<int64_t>(head + mp * rep) * dim + st * 16 + 8 * h);
+      qf[mp][st] = __builtin_bit_cast(bf16x8, z);
+    }
+    m[mp] = kNegBig;
+    l[mp] = 0.f;
+#pragma unroll
+    for (int vt = 0; vt < NV; ++vt)
+#pragma unroll
+      for (int i = 0; i < 16; ++i) O[mp][vt][i] = 0.f;
   }
-  float m = kNegBig, l = 0.f;
   if (use_sink) {   // log2 units, like the scores
-    m = a.sink_val != nullptr ? a.sink_val[head] * 1.44269504088896341f : 0.f;
-    l = 1.f;
+    m[0] = a.sink_val != nullptr ? a.sink_val[head] * 1.44269504088896341f : 0.f;
+    l[0] = 1.f;
   }
-  f32x16 O[NV];
-#pragma unroll
-  for (int vt = 0; vt < NV; ++vt)
-#pragma unroll
-    for (int i = 0; i < 16; ++i) O[vt][i] = 0.f;
   // the pages this workgroup walks, copied to LDS once: a key's page is then an LDS read and a
   // tile costs one global round trip, not two dependent ones
   const int* btg = a.block_tables + static_cast<int64_t>(s) * a.bt_width;
@@ -351,7 +493,7 @@ sink_attention_mfma_kernel(__bf16* __restrict__ out, const __bf16* __restrict__ 
   const bool bt_lds = npages <= kBtLds;
   if (bt_lds)
     for (int i = tid; i < npages; i += 256) lds_bt[i] = btg[page0 + i];
-  auto page_of = [&](int idx) -> int64_t { return bt_lds ? lds_bt[idx - page0] : btg[idx]; };
+  auto page_of = [&](int idx) -> int64_t { return bt_lds && idx >= page0 ? lds_bt[idx - page0] : btg[idx]; };
   // Staging plan of this thread, fixed for the whole loop: which 16-byte chunks of a K tile
   // (key, 8-channel group) and of a V^T tile (channel, 8-key group) it moves.  The page size is
   // a power of two (host-checked), so a key's page and offset are a shift and a mask.
@@ -368,20 +510,24 @@ sink_attention_mfma_kernel(__bf16* __restrict__ out, const __bf16* __restrict__ 
     k_src[c] = c8 * 8;
     k_dst[c] = key * KS + c8 * 8;
   }
-  const __bf16* kbase = k_cache + static_cast<int64_t>(g) * bs * dim;
-  const __bf16* vbase = v_cache + static_cast<int64_t>(g) * vdim * bs;
-  const int64_t kpage = static_cast<int64_t>(G) * bs * dim, vpage = static_cast<int64_t>(G) * vdim * bs;
-  for (int k0 = kbeg; k0 < kend; k0 += kKeys) {
+  const __bf16* kbase = k_cache + static_cast<int64_t>(NMAP * g) * bs * dim;
+  const __bf16* vbase = v_cache + static_cast<int64_t>(gv) * vdim * bs;
+  const int64_t kpage = static_cast<int64_t>(G) * bs * dim, vpage = static_cast<int64_t>(GV) * vdim * bs;
+  for (int k0 = part0 < kkeep ? part0 : kbeg; k0 < kend;
+       k0 = k0 + kKeys < kbeg && k0 + kKeys >= kkeep ? kbeg : k0 + kKeys) {
     __syncthreads();
 #pragma unroll
     for (int c = 0; c < KC; ++c) {
       if (k_key[c] < 0) continue;
       const int tk = k0 + k_key[c];
-      u32x4 z = {0u, 0u, 0u, 0u};
-      if (tk < kend)
-        z = *reinterpret_cast<const u32x4*>(kbase + page_of(tk >> bshift) * kpage +
-                                            (tk & bmask) * dim + k_src[c]);
-      *reinterpret_cast<u32x4*>(lds_k + k_dst[c]) = z;
+#pragma unroll
+      for (int mp = 0; mp < NMAP; ++mp) {
+        u32x4 z = {0u, 0u, 0u, 0u};
+        if (tk < kend)
+          z = *reinterpret_cast<const u32x4*>(kbase + page_of(tk >> bshift) * kpage +
+                                              (mp * bs + (tk & bmask)) * dim + k_src[c]);
+        *reinterpret_cast<u32x4*>(lds_k + mp * kKeys * KS + k_dst[c]) = z;
+      }
     }
 #pragma unroll
     for (int c = 0; c < VC; ++c) {
@@ -410,62 +556,65 @@ sink_attention_mfma_kernel(__bf16* __restrict__ out, const __bf16* __restrict__ 
     }
     __syncthreads();
     if (!wave_on) continue;
-    f32x16 S;
 #pragma unroll
-    for (int i = 0; i < 16; ++i) S[i] = 0.f;
+    for (int mp = 0; mp < NMAP; ++mp) {
+      f32x16 S;
 #pragma unroll
-    for (int st = 0; st < ND; ++st) {
-      if (st < nd) {
-        const bf16x8 kf = *reinterpret_cast<const bf16x8*>(lds_k + r * KS + st * 16 + 8 * h);
-        S = __builtin_amdgcn_mfma_f32_32x32x16_bf16(kf, qf[st], S, 0, 0, 0);
+      for (int i = 0; i < 16; ++i) S[i] = 0.f;
+#pragma unroll
+      for (int st = 0; st < ND; ++st) {
+        if (st < nd) {
+          const bf16x8 kf = *reinterpret_cast<const bf16x8*>(lds_k + (mp * kKeys + r) * KS + st * 16 + 8 * h);
+          S = __builtin_amdgcn_mfma_f32_32x32x16_bf16(kf, qf[mp][st], S, 0, 0, 0);
+        }
       }
-    }
-    // scores in log2 units (scale * log2 e folded into one multiply; the sink's score 0 stays 0);
-    // only tiles that reach the wave's causal edge or the end of the keys are masked
-    float tmax = kNegBig;
-    // (a masked score is -inf, the running maximum starts at the finite kNegBig: a column whose
-    // window has not begun yet keeps weight exp2(-inf) = 0 on every key of the tile)
-    if (k0 + kKeys - 1 > qpos_first || k0 + kKeys > kend || k0 <= edge_lo) {
+      // scores in log2 units (scale * log2 e folded into one multiply; the sink's score 0 stays 0);
+      // only tiles that reach the wave's causal edge or the end of the keys are masked
+      float tmax = kNegBig;
+      // (a masked score is -inf, the running maximum starts at the finite kNegBig: a column whose
+      // window has not begun yet keeps weight exp2(-inf) = 0 on every key of the tile)
+      if (k0 + kKeys - 1 > qpos_first || k0 + kKeys > kend || k0 <= edge_lo) {
+#pragma unroll
+        for (int i = 0; i < 16; ++i) {
+          const int key = k0 + 8 * (i >> 2) + 4 * h + (i & 3);
+          S[i] = (key <= qpos && (key >= qlow || key < a.keep) && key < kend) ? S[i] * scale2 : -INFINITY;
+          tmax = fmaxf(tmax, S[i]);
+        }
+      } else {
+#pragma unroll
+        for (int i = 0; i < 16; ++i) {
+          S[i] *= scale2;
+          tmax = fmaxf(tmax, S[i]);
+        }
+      }
+      tmax = fmaxf(tmax, __shfl_xor(tmax, 32, kWave));
+      const float m_new = fmaxf(m[mp], tmax);
+      const float alpha = __builtin_amdgcn_exp2f(m[mp] - m_new);
+      float psum = 0.f;
 #pragma unroll
       for (int i = 0; i < 16; ++i) {
-        const int key = k0 + 8 * (i >> 2) + 4 * h + (i & 3);
-        S[i] = (key <= qpos && key >= qlow && key < kend) ? S[i] * scale2 : -INFINITY;
-        tmax = fmaxf(tmax, S[i]);
+        S[i] = __builtin_amdgcn_exp2f(S[i] - m_new);   // masked scores: exp2(-inf) = 0
+        psum += S[i];
       }
-    } else {
+      psum += __shfl_xor(psum, 32, kWave);
+      l[mp] = l[mp] * alpha + psum;
+      m[mp] = m_new;
+      bf16x8 pk[2];
 #pragma unroll
-      for (int i = 0; i < 16; ++i) {
-        S[i] *= scale2;
-        tmax = fmaxf(tmax, S[i]);
-      }
-    }
-    tmax = fmaxf(tmax, __shfl_xor(tmax, 32, kWave));
-    const float m_new = fmaxf(m, tmax);
-    const float alpha = __builtin_amdgcn_exp2f(m - m_new);
-    float psum = 0.f;
+      for (int st = 0; st < 2; ++st)
 #pragma unroll
-    for (int i = 0; i < 16; ++i) {
-      S[i] = __builtin_amdgcn_exp2f(S[i] - m_new);   // masked scores: exp2(-inf) = 0
-      psum += S[i];
-    }
-    psum += __shfl_xor(psum, 32, kWave);
-    l = l * alpha + psum;
-    m = m_new;
-    bf16x8 pk[2];
+        for (int j = 0; j < 8; ++j) pk[st][j] = static_cast<__bf16>(S[8 * st + j]);
 #pragma unroll
-    for (int st = 0; st < 2; ++st)
+      for (int vt = 0; vt < NV; ++vt) {
+        if (vt < nv) {
 #pragma unroll
-      for (int j = 0; j < 8; ++j) pk[st][j] = static_cast<__bf16>(S[8 * st + j]);
+          for (int i = 0; i < 16; ++i) O[mp][vt][i] *= alpha;
 #pragma unroll
-    for (int vt = 0; vt < NV; ++vt) {
-      if (vt < nv) {
-#pragma unroll
-        for (int i = 0; i < 16; ++i) O[vt][i] *= alpha;
-#pragma unroll
-        for (int st = 0; st < 2; ++st) {
-          const bf16x8 vf = *reinterpret_cast<const bf16x8*>(lds_v + (vt * 32 + r) * kVStride +
-                                                             16 * st + 8 * h);
-          O[vt] = __builtin_amdgcn_mfma_f32_32x32x16_bf16(vf, pk[st], O[vt], 0, 0, 0);
+          for (int st = 0; st < 2; ++st) {
+            const bf16x8 vf = *reinterpret_cast<const bf16x8*>(lds_v + (vt * 32 + r) * kVStride +
+                                                               16 * st + 8 * h);
+            O[mp][vt] = __builtin_amdgcn_mfma_f32_32x32x16_bf16(vf, pk[st], O[mp][vt], 0, 0, 0);
+          }
         }
       }
     }
@@ -478,24 +627,71 @@ sink_attention_mfma_kernel(__bf16* __restrict__ out, const __bf16* __restrict__ 
     for (int vt = 0; vt < NV; ++vt)
       if (vt < nv)
 #pragma unroll
-        for (int i = 0; i < 16; ++i) po[vt * 32 + 8 * (i >> 2) + 4 * h + (i & 3)] = O[vt][i];
+        for (int i = 0; i < 16; ++i) po[vt * 32 + 8 * (i >> 2) + 4 * h + (i & 3)] = O[0][vt][i];
     if (h == 0) {
-      po[vdim] = m * 0.693147180559945309f;   // the combine kernel works in natural-log units
-      po[vdim + 1] = l;
+      po[vdim] = m[0] * 0.693147180559945309f;   // the combine kernel works in natural-log units
+      po[vdim + 1] = l[0];
     }
     return;
   }
-  const float inv = (l > 0.f ? 1.0f / l : 0.f) * head_gate_of<__bf16>(a, qrow, head);
-  __bf16* o = out + (qrow * H + head) * vdim;
+  if (NMAP == 2) {
+    // both lanes of a column (halves h) take part in the sum; they are valid together
+    const float i1 = l[0] > 0.f ? 1.0f / l[0] : 0.f;
+    const float i2 = l[NMAP - 1] > 0.f ? a.lam / l[NMAP - 1] : 0.f;
+    float ss = 0.f;
+#pragma unroll
+    for (int vt = 0; vt < NV; ++vt)
+      if (vt < nv)
+#pragma unroll
+        for (int i = 0; i < 16; ++i) {
+          const float o = O[0][vt][i] * i1 - O[NMAP - 1][vt][i] * i2;
+          O[0][vt][i] = o;
+          ss += o * o;
+        }
+    ss += __shfl_xor(ss, 32, kWave);
+    const float f = a.post / sqrtf(ss / static_cast<float>(vdim) + a.eps);
+    const int ho = g * rep + col % rep;
+    const __bf16* gt = a.gate != nullptr ? static_cast<const __bf16*>(a.gate) + qrow * a.gate_stride +
+                                               static_cast<int64_t>(ho) * vdim : nullptr;
+    __bf16* o = static_cast<__bf16*>(out) + (qrow * (H / 2) + ho) * vdim;
+#pragma unroll
+    for (int vt = 0; vt < NV; ++vt) {
+      if (vt < nv) {
+#pragma unroll
+        for (int i4 = 0; i4 < 4; ++i4) {
+          const int ch = vt * 32 + 8 * i4 + 4 * h;
+          bf16x4 gv4, e;
+          if (gt != nullptr) gv4 = *reinterpret_cast<const bf16x4*>(gt + ch);
+#pragma unroll
+          for (int j = 0; j < 4; ++j)
+            e[j] = static_cast<__bf16>(O[0][vt][4 * i4 + j] * f *
+                                       (gt != nullptr ? sigmoidf_(static_cast<float>(gv4[j])) : 1.0f));
+          *reinterpret_cast<bf16x4*>(o + ch) = e;
+        }
+      }
+    }
+    return;
+  }
+  const float inv = (l[0] > 0.f ? 1.0f / l[0] : 0.f) * head_gate_of<__bf16>(a, qrow, head);
+  const int64_t o = (qrow * H + head) * vdim;
 #pragma unroll
   for (int vt = 0; vt < NV; ++vt) {
     if (vt < nv) {
 #pragma unroll
       for (int i4 = 0; i4 < 4; ++i4) {
-        bf16x4 e;
+        const int64_t at = o + vt * 32 + 8 * i4 + 4 * h;
+        if (a.out_f32) {
+          typedef __attribute__((ext_vector_type(4))) float f32x4;
+          f32x4 e;
 #pragma unroll
-        for (int j = 0; j < 4; ++j) e[j] = static_cast<__bf16>(O[vt][4 * i4 + j] * inv);
-        *reinterpret_cast<bf16x4*>(o + vt * 32 + 8 * i4 + 4 * h) = e;
+          for (int j = 0; j < 4; ++j) e[j] = O[0][vt][4 * i4 + j] * inv;
+          *reinterpret_cast<f32x4*>(static_cast<float*>(out) + at) = e;
+        } else {
+          bf16x4 e;
+#pragma unroll
+          for (int j = 0; j < 4; ++j) e[j] = static_cast<__bf16>(O[0][vt][4 * i4 + j] * inv);
+          *reinterpret_cast<bf16x4*>(static_cast<__bf16*>(out) + at) = e;
+        }
       }
     }
   }
@@ -519,9 +715,21 @@ int opt_in_smem(K kernel, size_t smem, size_t* opted) {
 }
 
 // partitions a decode row can touch: all of its context, or the ones its window overlaps
-int decode_parts(int max_decode_kv, int window) {
+int decode_parts(int max_decode_kv, int window, int keep) {
   const int all = (max_decode_kv + kPartTokens - 1) / kPartTokens;
-  return window > 0 ? min(all, (window + kPartTokens - 1) / kPartTokens + 1) : all;
+  return window > 0 ? min(all, (window + kPartTokens - 1) / kPartTokens + 1 +
+                                   (keep + kPartTokens - 1) / kPartTokens)
+                    : all;
+}
+
+template <typename T>
+void launch_combine(void* out, const AttnArgs& a, int num_decode, hipStream_t st) {
+  if (a.pair)
+    hipLaunchKernelGGL(pair_attention_combine_kernel<T>, dim3(num_decode, a.H / 2), dim3(kWave), 0,
+                       st, static_cast<T*>(out), a);
+  else
+    hipLaunchKernelGGL(sink_attention_combine_kernel<T>, dim3(num_decode, a.H), dim3(kWave), 0, st,
+                       out, a);
 }
 
 template <typename T>
@@ -536,20 +744,19 @@ int launch_rows(void* out, const void* q, const void* k_cache, const void* v_cac
   if (num_tiles > 0) {
     if (int rc = opt_in_smem(sink_attention_rows_kernel<T, false>, smem, &opted_p)) return rc;
     hipLaunchKernelGGL((sink_attention_rows_kernel<T, false>), dim3(num_tiles * 4, a.H), dim3(256),
-                       smem, st, static_cast<T*>(out), static_cast<const T*>(q),
+                       smem, st, out, static_cast<const T*>(q),
                        static_cast<const T*>(k_cache), static_cast<const T*>(v_cache), a);
   }
   if (num_decode > 0) {
     if (int rc = opt_in_smem(sink_attention_rows_kernel<T, true>, smem, &opted_d)) return rc;
-    const int parts = decode_parts(max_decode_kv, a.window);
+    const int parts = decode_parts(max_decode_kv, a.window, a.keep);
     if (parts > a.max_parts || parts < 1) return -1;
     const int head_blocks = (a.H / a.G + kRows - 1) / kRows;
     hipLaunchKernelGGL((sink_attention_rows_kernel<T, true>),
                        dim3(num_decode, a.G * head_blocks, parts),
-                       dim3(256), smem, st, static_cast<T*>(out), static_cast<const T*>(q),
+                       dim3(256), smem, st, out, static_cast<const T*>(q),
                        static_cast<const T*>(k_cache), static_cast<const T*>(v_cache), a);
-    hipLaunchKernelGGL(sink_attention_combine_kernel<T>, dim3(num_decode, a.H), dim3(kWave), 0, st,
-                       static_cast<T*>(out), a);
+    launch_combine<T>(out, a, num_decode, st);
   }
   return static_cast<int>(hipGetLastError());
 }
@@ -558,42 +765,70 @@ template <int ND, int NV>
 void launch_mfma(void* out, const void* q, const void* k_cache, const void* v_cache, AttnArgs a,
                  int num_tiles, int num_decode, int parts, hipStream_t st) {
   const int chunks = (kTileTokens * (a.H / a.G) + 127) / 128;
-  if (num_tiles > 0)
+  if (num_tiles > 0 && !a.pair)
     hipLaunchKernelGGL((sink_attention_mfma_kernel<ND, NV, false>), dim3(num_tiles, a.G, chunks),
-                       dim3(256), 0, st, static_cast<__bf16*>(out), static_cast<const __bf16*>(q),
+                       dim3(256), 0, st, out, static_cast<const __bf16*>(q),
                        static_cast<const __bf16*>(k_cache), static_cast<const __bf16*>(v_cache), a);
   if (num_decode > 0) {
     hipLaunchKernelGGL((sink_attention_mfma_kernel<ND, NV, true>), dim3(num_decode, a.G, parts),
-                       dim3(256), 0, st, static_cast<__bf16*>(out), static_cast<const __bf16*>(q),
+                       dim3(256), 0, st, out, static_cast<const __bf16*>(q),
                        static_cast<const __bf16*>(k_cache), static_cast<const __bf16*>(v_cache), a);
-    hipLaunchKernelGGL(sink_attention_combine_kernel<__bf16>, dim3(num_decode, a.H), dim3(kWave),
-                       0, st, static_cast<__bf16*>(out), a);
+    launch_combine<__bf16>(out, a, num_decode, st);
   }
+}
+
+template <int ND, int NV>
+void launch_pair(void* out, const void* q, const void* k_cache, const void* v_cache, AttnArgs a,
+                 int num_tiles, hipStream_t st) {
+  const int chunks = (kTileTokens * (a.H / a.G) + 127) / 128;
+  hipLaunchKernelGGL((sink_attention_mfma_kernel<ND, NV, false, 2>),
+                     dim3(num_tiles, a.G / 2, chunks), dim3(256), 0, st, out,
+                     static_cast<const __bf16*>(q), static_cast<const __bf16*>(k_cache),
+                     static_cast<const __bf16*>(v_cache), a);
 }
 
 }  // namespace mixk
 
 using namespace mixk;
 
+extern "C" int mixk_diff_combine(void* out, const float* in, const void* gate, int64_t gate_stride,
+                                 int T_, int HO, int G, int vdim, float lam, float post, float eps,
+                                 int dtype, hipStream_t st) {
+  if (T_ <= 0) return 0;
+  if (HO <= 0 || G <= 0 || HO % G != 0 || vdim <= 0) return -1;
+  const int64_t waves = static_cast<int64_t>(T_) * HO;
+  MIXK_DISPATCH(dtype, hipLaunchKernelGGL(diff_combine_kernel<T>,
+                                          dim3(static_cast<unsigned>((waves + 3) / 4)), dim3(256),
+                                          0, st, static_cast<T*>(out), in,
+                                          static_cast<const T*>(gate), gate_stride, T_, HO, G, vdim,
+                                          lam, post, eps));
+  return static_cast<int>(hipGetLastError());
+}
+
 // Prefill tiles (64 query tokens each: tile_seq / tile_qoff) and decode sequences
 // [0, num_decode) (one query row each, row = seq_qstart[s]; partials in `part`
 // [num_decode, H, max_parts, vdim + 2] fp32).  use_mfma: bf16 matrix-core prefill kernel.
+// pair: H and G count both maps of differential attention, out is [T, H / 2, vdim] of the activation
+// dtype and gate [T, H / 2 * vdim]; needs use_mfma.  v_share: K heads per V head.
 extern "C" int mixk_sink_attention(void* out, const void* q, const void* k_cache,
                                    const void* v_cache, const int* block_tables, int bt_width,
                                    const int* seq_kvlen, const int* seq_qstart,
                                    const int* tile_seq, const int* tile_qoff, int num_tiles,
                                    int num_decode, int max_decode_kv, float* part, int max_parts,
                                    int H, int G, int dim, int vdim, int block_size, float scale,
-                                   int sink, const float* sink_val, int window,
-                                   const void* gate, int64_t gate_stride, int use_mfma, int dtype,
-                                   hipStream_t st) {
+                                   int sink, const float* sink_val, int window, int keep,
+                                   const void* gate, int64_t gate_stride, int v_share,
+                                   int64_t q_stride, int out_f32, int pair, float lam, float post,
+                                   float eps, int use_mfma, int dtype, hipStream_t st) {
   if (num_tiles <= 0 && num_decode <= 0) return 0;
-  if (vdim > 16 * kMaxVPer || G <= 0 || H % G != 0) return -1;
+  if (vdim > 16 * kMaxVPer || G <= 0 || H % G != 0 || v_share < 1 || G % v_share != 0) return -1;
+  if (pair && (!use_mfma || sink || v_share != 2)) return -1;
   int bs_shift = 0;
   while ((1 << bs_shift) < block_size) ++bs_shift;
   AttnArgs a{block_tables, seq_kvlen, seq_qstart, tile_seq, tile_qoff, part, sink ? sink_val : nullptr,
              bt_width, H, G, dim, vdim, block_size, sink, 0, max_parts, bs_shift, scale,
-             window > 0 ? window : 0, gate, gate_stride};
+             window > 0 ? window : 0, window > 0 ? max(keep, 0) : 0, v_share, q_stride, out_f32,
+             pair, lam, post, eps, gate, gate_stride};
   int rc = 0;
   if (use_mfma) {
     if (dtype != 0 || dim % 16 || vdim % 32 || dim > 256 || vdim > 256 || block_size < 8 ||
@@ -601,7 +836,7 @@ extern "C" int mixk_sink_attention(void* out, const void* q, const void* k_cache
       return -1;
     // decode columns = the query heads of one KV head: they must fit one workgroup
     const int nd_mfma = (H / G <= 128) ? num_decode : 0;
-    const int parts = decode_parts(max_decode_kv, a.window);
+    const int parts = decode_parts(max_decode_kv, a.window, a.keep);
     if (nd_mfma > 0 && (parts > max_parts || parts < 1)) return -1;
     if (dim <= 64 && vdim <= 64)
       launch_mfma<4, 2>(out, q, k_cache, v_cache, a, num_tiles, nd_mfma, parts, st);
@@ -609,6 +844,16 @@ extern "C" int mixk_sink_attention(void* out, const void* q, const void* k_cache
       launch_mfma<8, 4>(out, q, k_cache, v_cache, a, num_tiles, nd_mfma, parts, st);
     else
       launch_mfma<16, 8>(out, q, k_cache, v_cache, a, num_tiles, nd_mfma, parts, st);
+    if (pair && num_tiles > 0) {
+      if (dim <= 64 && vdim <= 64)
+        launch_pair<4, 2>(out, q, k_cache, v_cache, a, num_tiles, st);
+      else if (dim <= 64 && vdim <= 128)
+        launch_pair<4, 4>(out, q, k_cache, v_cache, a, num_tiles, st);
+      else if (dim <= 128 && vdim <= 128)
+        launch_pair<8, 4>(out, q, k_cache, v_cache, a, num_tiles, st);
+      else
+        launch_pair<16, 8>(out, q, k_cache, v_cache, a, num_tiles, st);
+    }
     rc = static_cast<int>(hipGetLastError());
     if (rc) return rc;
     num_tiles = 0;

@@ -204,6 +204,17 @@ def mfma_attention_ok(q, k_cache, v_cache) -> bool:
             and vdim <= 256 and bs >= 8 and bs & (bs - 1) == 0 and ATTENTION_MFMA)
 
 
+def _decode_partials(num_decode, heads, max_decode_kv, vdim, window, keep_first, device):
+    """Workspace of the partitioned decode attention (None without decode rows)."""
+    if num_decode <= 0:
+        return None
+    parts = max(1, -(-int(max_decode_kv) // DECODE_PART_TOKENS))
+    if window > 0:   # the window and the kept keys touch at most this many partitions
+        parts = min(parts, -(-window // DECODE_PART_TOKENS) + 1
+                    + -(-keep_first // DECODE_PART_TOKENS))
+    return torch.empty(num_decode, heads, parts, vdim + 2, dtype=torch.float32, device=device)
+
+
 def sink_attention(q, k_cache, v_cache, block_tables, seq_kvlen, seq_qstart, tile_seq, tile_qoff,
                    scale, sink=True, num_decode=0, max_decode_kv=0, sink_values=None, window=0,
                    gate=None, keep_first=0, out_dtype=None):
@@ -226,20 +237,14 @@ def sink_attention(q, k_cache, v_cache, block_tables, seq_kvlen, seq_qstart, til
                                    scale, sink, sink_values, window, gate, keep_first, out_dtype)
     out = torch.empty(q.shape[0], q.shape[1], v_cache.shape[2], dtype=out_dtype or q.dtype,
                       device=q.device)
-    part = None
-    if num_decode > 0:
-        parts = max(1, -(-int(max_decode_kv) // DECODE_PART_TOKENS))
-        if window > 0:   # the window touches at most this many partitions
-            parts = min(parts, -(-window // DECODE_PART_TOKENS) + 1
-                        + -(-keep_first // DECODE_PART_TOKENS))
-        part = torch.empty(num_decode, q.shape[1], parts, v_cache.shape[2] + 2,
-                           dtype=torch.float32, device=q.device)
+    part = _decode_partials(num_decode, q.shape[1], max_decode_kv, v_cache.shape[2], window,
+                            keep_first, q.device)
     if tile_seq.shape[0] > 0 or num_decode > 0:
         _native().sink_attention(out, q, k_cache, v_cache, block_tables, seq_kvlen, seq_qstart,
                                  tile_seq, tile_qoff, scale, sink, num_decode,
                                  max(1, int(max_decode_kv)), part,
                                  mfma_attention_ok(q, k_cache, v_cache), sink_values, window, gate,
-                                 keep_first)
+                                 keep_first, None)
     return out
 
 
@@ -270,6 +275,18 @@ def differential_attention(q, k_cache, v_cache, block_tables, seq_kvlen, seq_qst
     [nb, 2 G, BS, d] hold the heads in the order (KV head, map, head of the group), v_cache
     [nb, G, dv, BS] is shared by the maps; returns ``diff_combine`` of the two
     ([T, H * dv], q's dtype).  Batch layout, window and ``keep_first`` as in ``sink_attention``."""
+    if q.is_cuda and mfma_attention_ok(q, k_cache, v_cache):
+        # both maps in one workgroup over one staged V tile; decode rows joined by the combine kernel
+        T, H, dv = q.shape[0], q.shape[1] // 2, v_cache.shape[2]
+        keep_first = int(keep_first) if window > 0 else 0
+        out = torch.empty(T, H, dv, dtype=q.dtype, device=q.device)
+        part = _decode_partials(num_decode, 2 * H, max_decode_kv, dv, window, keep_first, q.device)
+        if tile_seq.shape[0] > 0 or num_decode > 0:
+            _native().sink_attention(out, q, k_cache, v_cache, block_tables, seq_kvlen, seq_qstart,
+                                     tile_seq, tile_qoff, scale, False, num_decode,
+                                     max(1, int(max_decode_kv)), part, True, None, int(window), gate,
+                                     keep_first, [float(lam), 1.0 - float(diff), float(eps)])
+        return out.view(T, H * dv)
     a = sink_attention(q, k_cache, v_cache, block_tables, seq_kvlen, seq_qstart, tile_seq, tile_qoff,
                        scale, False, num_decode, max_decode_kv, window=window,
                        keep_first=keep_first, out_dtype=torch.float32)
