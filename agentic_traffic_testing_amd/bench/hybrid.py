@@ -1,12 +1,12 @@
 """Prefill and decode throughput of the hybrid decoders (Ledazen, Soselix, Semezen, Lovapel,
-Kolotar) next to the models of the same layer geometry - Llama, and for the later families also the
+Kolotar, Tofodra) next to the models of the same layer geometry - Llama, and for the later families also the
 closest earlier hybrid ones (softmax + recurrent mixers on the same cache and kernels) - through the serving
 engine (scheduler, paged cache / state slots, kernels).
 
 Random-init weights, synthetic token ids.  Per model and shape:
   prefill  - B prompts of P tokens admitted together, one generated token each: prompt tok/s
   decode   - the same B sequences generating N more tokens: generated tok/s
-``python bench.py --hybrid [ledazen|soselix|semezen|lovapel|kolotar]`` prints one JSON line per measurement.
+``python bench.py --hybrid [ledazen|soselix|semezen|lovapel|kolotar|tofodra]`` prints one JSON line per measurement.
 """
 from __future__ import annotations
 
@@ -29,8 +29,11 @@ LOVAPEL = (("lovapel-small", "semezen-small", "small"),
 KOLOTAR = tuple((f"kolotar-{s}", f"lovapel-{s}", f"soselix-{s}",
                  "small" if s == "small" else f"llama-{s}")
                 for s in ("small", "3b-slice", "8b-slice"))
+TOFODRA = tuple((f"tofodra-{s}", f"kolotar-{s}", f"soselix-{s}",
+                 "small" if s == "small" else f"llama-{s}")
+                for s in ("small", "3b-slice", "8b-slice"))
 FAMILIES = {"ledazen": PAIRS, "soselix": SOSELIX, "semezen": SEMEZEN, "lovapel": LOVAPEL,
-            "kolotar": KOLOTAR}
+            "kolotar": KOLOTAR, "tofodra": TOFODRA}
 
 
 def _engine(model: str, device: str, dtype: str, max_len: int, seqs: int, budget: int):

@@ -179,11 +179,10 @@ def silu_glu(h, st, p):
 
 def route(z, top, scale):
     """One token's router logits -> (the ``top`` with the largest sigmoid scores, weights, the gap
-    in score to the best one left out)."""
-    s = torch.sigmoid(z)
-    srt = torch.sort(s, descending=True)
+    between the logits of the last one chosen and the best one left out)."""
+    srt = torch.sort(z, descending=True)     # the sigmoid keeps the order
     gap = float(srt.values[top - 1] - srt.values[top]) if z.shape[0] > top else 1e9
-    w = srt.values[:top]
+    w = torch.sigmoid(srt.values[:top])
     return srt.indices[:top], w / (w.sum() + 1e-20) * scale, gap
 
 
