@@ -71,7 +71,8 @@ retention_chunk_kernel(RetArgs a) {
   float* Ks = Qs + kChunk * DS;                 // [64][DS]
   float* St = Ks + kChunk * DS;                 // [64 columns][DS]: S^T
   float* Vt = St + kRetCols * DS;               // [64 columns][kTokStride]: V^T
-  float* Ps = Vt + kRetCols * kTokStride;       // [64][kTokStride]: masked, decayed scores
+  float* Vd = Vt + kRetCols * kTokStride;       // the same, decayed to the end of the chunk
+  float* Ps = Vd + kRetCols * kTokStride;       // [64][kTokStride]: masked, decayed scores
   float* pw = Ps + kChunk * kTokStride;         // [kChunk + 1]
   const int s = a.seq0 + blockIdx.x, h = blockIdx.y, tid = threadIdx.x;
   const int slot = a.seq_slot[s];
@@ -85,9 +86,8 @@ retention_chunk_kernel(RetArgs a) {
   const T* vp = static_cast<const T*>(a.v) + static_cast<int64_t>(h) * dv + c0;
   float* st = a.state + (static_cast<int64_t>(slot) * H + h) * dk * dv;
   if (tid <= kChunk) pw[tid] = a.powers[h * (kChunk + 1) + tid];
-  // channels past dk and columns past dv stay zero in every staged array
+  // channels past dk stay zero in every staged array (V's columns past dv are staged as zeros)
   for (int i = tid; i < kChunk * DS; i += 256) Qs[i] = Ks[i] = St[i] = 0.f;
-  for (int i = tid; i < kRetCols * kTokStride; i += 256) Vt[i] = 0.f;
   // this wave's blocks of S: rows db 32 .. + 31, columns cb 32 .. + 31
   rf32x16 S[SB];
   const bool fresh = a.positions[first] == 0;
@@ -232,11 +232,16 @@ retention_chunk_kernel(RetArgs a) {
         }
       }
     }
+    const float decay_to_end = pw[max(nt - 1 - (tid & 63), 0)];   // of this thread's V token
 #pragma unroll
     for (int m = 0; m < 2; ++m) {
       const int it = tid + m * 256, tt = it & 63, cg = (it >> 6) * 8;
 #pragma unroll
-      for (int e = 0; e < 8; ++e) Vt[(cg + e) * kTokStride + tt] = static_cast<float>(rv[m][e]);
+      for (int e = 0; e < 8; ++e) {
+        const float v = static_cast<float>(rv[m][e]);
+        Vt[(cg + e) * kTokStride + tt] = v;
+        Vd[(cg + e) * kTokStride + tt] = v * decay_to_end;
+      }
     }
     __syncthreads();
     if (t0 + kChunk < n) fetch(t0 + kChunk);   // in flight during the products below
@@ -315,13 +320,12 @@ retention_chunk_kernel(RetArgs a) {
       const int blk = w + 4 * b, db = blk % NDB, sc = blk / NDB;
       if (blk < 2 * NDB) {   // wave-uniform
         const float* kr = Ks + (4 * hf) * DS + db * 32 + r;
-        const float* vr = Vt + (sc * 32 + r) * kTokStride + 4 * hf;
+        const float* vr = Vd + (sc * 32 + r) * kTokStride + 4 * hf;
 #pragma unroll
         for (int j = 0; j < kChunk; j += 8) {
           const rf32x4 va = *reinterpret_cast<const rf32x4*>(vr + j);
 #pragma unroll
-          for (int e = 0; e < 4; ++e)
-            S[b] = mfma_f32(kr[(j + e) * DS], va[e] * pw[max(nt - 1 - j - 4 * hf - e, 0)], S[b]);
+          for (int e = 0; e < 4; ++e) S[b] = mfma_f32(kr[(j + e) * DS], va[e], S[b]);
         }
       }
     }
@@ -435,7 +439,7 @@ retention_step_kernel(RetArgs a) {
 
 template <typename T, int DK, bool VEC>
 int launch_chunk(const RetArgs& a, int seqs, hipStream_t st) {
-  constexpr size_t smem = sizeof(float) * (3 * kChunk * (DK + 4) + 2 * kChunk * kTokStride + kChunk + 4);
+  constexpr size_t smem = sizeof(float) * (3 * kChunk * (DK + 4) + 3 * kChunk * kTokStride + kChunk + 4);
   static bool opted = false;
   if (smem > 48 * 1024 && !opted) {
     hipError_t e = hipFuncSetAttribute(
