@@ -880,3 +880,128 @@ def test_route_by_logit(E, top):
     want = mref.moe_route(logits, top, "logit")
     assert torch.equal(got[0].cpu(), want[0])
     assert torch.allclose(got[1].cpu(), want[1], atol=1e-6, rtol=1e-5)
+
+
+# ---- retention, differential attention, windows that keep the first tokens ------------------------
+@pytest.mark.parametrize("dt", DTYPES)
+@pytest.mark.parametrize("H,dk,dv,nf", [(3, 64, 64, 32), (2, 128, 128, 32), (4, 24, 20, 8), (2, 32, 80, 16),
+                                        (1, 256, 64, 64), (3, 48, 72, 0), (2, 9, 5, 2), (1, 1, 1, 0)])
+def test_retention(dt, H, dk, dv, nf):
+    torch.manual_seed(dk + dv)
+    lens, starts, slots = [1, 1, 70, 2, 64, 129, 200, 3], [5, 0, 0, 11, 0, 64, 7, 0], [3, 1, 0, 2, -1, 5, 4, 6]
+    md = ragged(lens, starts, slots, width=24)
+    T = int(md["seq_qstart"][-1])
+    P = torch.randn(T, 2 * H * dk + H * dv + 24).to(dt)
+    state = torch.randn(8, H, dk, dv)
+    state_g = state.cuda()
+    tab = (mref.rotary_table(md["positions"], mx.inv_freq(2 * nf, 1000.0, "cpu")) if nf else
+           torch.zeros(T, 0))
+    pw = mx.retention_powers([0.9, 0.97, 0.999, 0.5][:H], "cpu")
+
+    def cut(X):
+        return (X[:, 8:8 + H * dk], X[:, 8 + H * dk:8 + 2 * H * dk],
+                X[:, 8 + 2 * H * dk:8 + 2 * H * dk + H * dv])
+
+    g = cuda(md)
+    a = mref.retention(*cut(P), pw[:, 1], tab, state, md["positions"], md["seq_qstart"],
+                       md["seq_slot"], H, dk, dv)
+    b = mx.retention(*cut(P.cuda()), pw.cuda(), tab.cuda(), state_g, g["positions"], g["seq_qstart"],
+                     g["seq_slot"], H, dk, dv, 2)
+    live = torch.ones(T, dtype=torch.bool)
+    live[int(md["seq_qstart"][4]):int(md["seq_qstart"][5])] = False
+    scale = float(a.abs().max())
+    assert float((a - b.cpu())[live].abs().max()) < 1e-5 * scale      # fp32 inside for both dtypes
+    assert float((state - state_g.cpu()).abs().max()) < 1e-5 * float(state.abs().max())
+
+
+@pytest.mark.parametrize("dt", DTYPES)
+@pytest.mark.parametrize("H,G,d,dv,window,keep", [(4, 2, 32, 64, 40, 5), (6, 1, 16, 32, 0, 0),
+                                                  (2, 2, 64, 128, 150, 140), (8, 4, 12, 20, 17, 30),
+                                                  (3, 3, 80, 96, 130, 2), (2, 1, 48, 160, 9, 1)])
+def test_differential_attention(dt, H, G, d, dv, window, keep):
+    """Decode rows, portions and pages in one ragged batch; the pair form and the two-step path."""
+    torch.manual_seed(H * d)
+    lens, starts = [1, 1, 1, 37, 2, 130], [0, 290, 128, 0, 140, 60]
+    md = ragged(lens, starts, [0, 1, 2, 3, 4, 5], width=24)
+    T, nb = int(md["seq_qstart"][-1]), md["num_pages"]
+    k, v = torch.randn(nb, 2 * G, 16, d).to(dt), torch.randn(nb, G, dv, 16).to(dt)
+    wide = torch.randn(T, 2 * H * d + H * dv + 32).to(dt)
+    tiles = md["tile_seq"] >= 3
+    md["tile_seq"], md["tile_qoff"] = md["tile_seq"][tiles], md["tile_qoff"][tiles]
+    g = cuda(md)
+
+    def run(w, kc, vc, m, **kw):
+        q = w[:, 8:8 + 2 * H * d].unflatten(1, (2 * H, d))
+        gate = w[:, 8 + 2 * H * d + 8:8 + 2 * H * d + 8 + H * dv]
+        return mx.differential_attention(q, kc, vc, m["block_tables"], m["seq_kvlen"], m["seq_qstart"],
+                                         m["tile_seq"], m["tile_qoff"], d ** -0.5, 0.7, 0.3, 1e-5,
+                                         gate, 3, 291, window, keep)
+
+    want, got = run(wide, k, v, md), run(wide.cuda(), k.cuda(), v.cuda(), g).cpu()
+    t = dict(atol=4e-2, rtol=4e-2) if dt == torch.bfloat16 else dict(atol=2e-5, rtol=1e-4)
+    assert torch.allclose(got.float(), want.float(), **t)
+    if dt == torch.bfloat16 and mx.mfma_attention_ok(wide[:, :d].view(T, 1, d), k, v):
+        was, mx.ATTENTION_MFMA = mx.ATTENTION_MFMA, False
+        try:
+            rows = run(wide.cuda(), k.cuda(), v.cuda(), g).cpu()
+        finally:
+            mx.ATTENTION_MFMA = was
+        assert torch.allclose(rows.float(), want.float(), **t)
+
+
+@pytest.mark.parametrize("dt", DTYPES)
+@pytest.mark.parametrize("d,dv", [(32, 64), (20, 28)])
+@pytest.mark.parametrize("window,keep", [(40, 5), (140, 300), (16, 16), (1, 1)])
+def test_kept_tokens_with_sink_and_gate(dt, d, dv, window, keep):
+    torch.manual_seed(window)
+    lens, starts = [1, 1, 37, 2, 130], [290, 0, 0, 140, 60]
+    md = ragged(lens, starts, [0, 1, 2, 3, 4], width=24)
+    T, nb, H, G = int(md["seq_qstart"][-1]), md["num_pages"], 4, 2
+    q, gate = torch.randn(T, H, d).to(dt), torch.randn(T, H).to(dt)
+    k, v = torch.randn(nb, G, 16, d).to(dt), torch.randn(nb, G, dv, 16).to(dt)
+    sink = torch.randn(H)
+    tiles = md["tile_seq"] >= 2
+    md["tile_seq"], md["tile_qoff"] = md["tile_seq"][tiles], md["tile_qoff"][tiles]
+    want = mref.sink_attention(q, k, v, md["block_tables"], md["seq_kvlen"], md["seq_qstart"], 0.2,
+                               True, sink, window, gate, keep)
+    g = cuda(md)
+    got = mx.sink_attention(q.cuda(), k.cuda(), v.cuda(), g["block_tables"], g["seq_kvlen"],
+                            g["seq_qstart"], g["tile_seq"], g["tile_qoff"], 0.2, True, 2, 291,
+                            sink.cuda(), window, gate.cuda(), keep)
+    assert torch.allclose(got.cpu().float(), want.float(), **tol(dt))
+
+
+@pytest.mark.parametrize("dt", DTYPES)
+def test_branch_scale_norms_and_glu(dt):
+    torch.manual_seed(4)
+    for W in (64, 100, 2048):
+        x = torch.randn(5, W)
+        y, w, s, wn = (torch.randn(*n).to(dt) for n in ((5, W), (W,), (W,), (W,)))
+        xg = x.cuda()
+        want = mref.norm_add_norm(x, y, w, wn, 1e-5, False, dt, s)
+        got = mx.norm_add_norm(xg, y.cuda(), w.cuda(), wn.cuda(), 1e-5, "rms", dt, post_scale=s.cuda())
+        assert torch.allclose(xg.cpu(), x, atol=2e-5, rtol=2e-5)
+        assert torch.allclose(got.cpu().float(), want.float(), **tol(dt))
+    for dv in (12, 64, 128, 136, 600):
+        o, gate, w = torch.randn(7, 3, dv), torch.randn(7, 3 * dv + 8).to(dt), torch.randn(dv).to(dt)
+        for wt in (None, w):
+            for act in ("silu", "sigmoid"):
+                want = mref.gated_rms_norm(o, gate[:, 8:], wt, 1e-5, act, dt)
+                got = mx.gated_rms_norm(o.cuda(), gate.cuda()[:, 8:], wt.cuda() if wt is not None else None,
+                                        1e-5, act, dt)
+                assert torch.allclose(got.cpu().float(), want.float(), **tol(dt)), (dv, act)
+    for n, off in ((64, 8), (33, 1), (2048, 0)):
+        p = (3.0 * torch.randn(6, 2 * n + off)).to(dt)
+        want = mref.clamped_gate_mul(p[:, off + n:], p[:, off:off + n], 2.0)
+        pg = p.cuda()
+        got = mx.clamped_gate_mul(pg[:, off + n:], pg[:, off:off + n], 2.0)
+        assert torch.allclose(got.cpu().float(), want.float(), **tol(dt))
+
+
+@pytest.mark.parametrize("E,top,scale", [(16, 4, 2.5), (5, 5, 1.0), (70, 3, 0.5), (300, 8, 7.0)])
+def test_scaled_sigmoid_route(E, top, scale):
+    logits = 2.0 * torch.randn(33, E, generator=torch.Generator().manual_seed(E))
+    idx, w = mx.moe_route(logits.cuda(), top, "sigmoid", renorm=True, scale=scale)
+    ri, rw = mref.moe_route(logits, top, "sigmoid", renorm=True, scale=scale)
+    assert torch.equal(idx.cpu(), ri) and torch.allclose(w.cpu(), rw, atol=1e-5, rtol=1e-5)
+    assert torch.allclose(w.cpu().sum(1), torch.full((33,), scale), rtol=1e-4)
